@@ -8,6 +8,7 @@
 //     holds no pair): an expert that runs on its weight times the input, the weight taken out of the two products;
 //   * add_row_bias: every row of a 32-bit matrix gets the same row added (the bias of an output product that
 //     accumulates into the residual stream);
+//   * squared_relu: max(x, 0)^2 of a product's 32-bit rows, in the activation type;
 //   * table_route: a token's experts read from a table by its id, each weighing 1 / top;
 //   * concat_rows: [a | b] side by side in the activation type, the input of a product over both.
 #include "common.h"
@@ -56,6 +57,14 @@ __global__ void add_row_bias_kernel(float* __restrict__ x, const TB* __restrict_
     const size_t idx = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
     if (idx >= total) return;
     x[idx] += to_float(bias[idx % H]);
+}
+
+template <typename TO>
+__global__ void squared_relu_kernel(const float* __restrict__ x, TO* __restrict__ out, size_t total) {
+    const size_t idx = static_cast<size_t>(blockIdx.x) * blockDim.x + threadIdx.x;
+    if (idx >= total) return;
+    const float v = fmaxf(x[idx], 0.f);
+    out[idx] = from_float<TO>(v * v);
 }
 
 __global__ void table_route_kernel(const int* __restrict__ table, const int* __restrict__ tokens, int* __restrict__ ids,
@@ -109,6 +118,17 @@ extern "C" int llme_add_row_bias(float* x, const void* bias, int bias_dtype, int
         hipLaunchKernelGGL((add_row_bias_kernel<float>), grid, dim3(256), 0, stream, x, static_cast<const float*>(bias), H, total);
     else if (bias_dtype == kBF16)
         hipLaunchKernelGGL((add_row_bias_kernel<bf16>), grid, dim3(256), 0, stream, x, static_cast<const bf16*>(bias), H, total);
+    else return kErrBadArgument;
+    return launch_status();
+}
+
+extern "C" int llme_squared_relu(const float* x, void* out, int out_dtype, size_t n, hipStream_t stream) {
+    if (n == 0) return 0;
+    const dim3 grid(static_cast<unsigned>((n + 255) / 256));
+    if (out_dtype == kF32)
+        hipLaunchKernelGGL((squared_relu_kernel<float>), grid, dim3(256), 0, stream, x, static_cast<float*>(out), n);
+    else if (out_dtype == kBF16)
+        hipLaunchKernelGGL((squared_relu_kernel<bf16>), grid, dim3(256), 0, stream, x, static_cast<bf16*>(out), n);
     else return kErrBadArgument;
     return launch_status();
 }

@@ -52,7 +52,14 @@ typedef __attribute__((ext_vector_type(4))) unsigned u32x4;
 constexpr int kBufferFlags = 0x00020000;
 
 enum OutMode : int { kStoreF32 = 0, kAddF32 = 1, kStoreBF16 = 2, kAtomicF32 = 3, kGatedBF16 = 4, kRopeCache = 5,
-                     kGatedReluBF16 = 6, kGatedGeluBF16 = 7, kGatedExtraBF16 = 8 };
+                     kGatedReluBF16 = 6, kGatedGeluBF16 = 7, kGatedExtraBF16 = 8, kSquaredReluBF16 = 9 };
+// Stored in bfloat16 one value a column: as it is, or the square of its positive part (kSquaredReluBF16).
+constexpr bool is_stored_bf16(int mode) { return mode == kStoreBF16 || mode == kSquaredReluBF16; }
+template <int MODE> __device__ __forceinline__ float stored_value(float v) {
+    if (MODE != kSquaredReluBF16) return v;
+    v = fmaxf(v, 0.f);
+    return v * v;
+}
 // The gated outputs: act(gate) * up with act = SiLU (kGatedBF16), the rectifier (kGatedReluBF16) or the tanh form of
 // GELU (kGatedGeluBF16); kGatedExtraBF16: SiLU or a clamped swish with biases on gate and up (GateExtra).
 constexpr bool is_gated(int mode) {
@@ -315,7 +322,7 @@ __device__ __forceinline__ void tile_epilogue(f32x4 (&acc)[WMT][WNT], unsigned c
                 const int unit = (n0 + (piece / 2) * 32) / 2 + (piece % 2) * 8;
                 *reinterpret_cast<bf16x8*>(static_cast<bf16*>(out) + static_cast<size_t>(m) * (N / 2) + unit) = o;
             }
-        } else if (MODE == kStoreBF16) {
+        } else if (is_stored_bf16(MODE)) {
             constexpr int PER_ROW = BN / 8;
             for (int idx = tid; idx < HB * PER_ROW; idx += NT) {
                 const int row = idx / PER_ROW, col = (idx % PER_ROW) * 8;
@@ -324,7 +331,7 @@ __device__ __forceinline__ void tile_epilogue(f32x4 (&acc)[WMT][WNT], unsigned c
                 const float* sp = stage + row * SS + col;
                 bf16x8 o;
 #pragma unroll
-                for (int e = 0; e < 8; ++e) o[e] = static_cast<__bf16>(sp[e]);
+                for (int e = 0; e < 8; ++e) o[e] = static_cast<__bf16>(stored_value<MODE>(sp[e]));
                 *reinterpret_cast<bf16x8*>(static_cast<bf16*>(out) + static_cast<size_t>(m) * N + n) = o;
             }
         } else if (MODE == kAddF32 && PASSES == 1 && AHEAD) {
@@ -394,7 +401,7 @@ __device__ __forceinline__ void tile_epilogue(f32x4 (&acc)[WMT][WNT], unsigned c
                     if (MODE == kStoreF32) static_cast<float*>(out)[idx] = v;
                     else if (MODE == kAddF32) static_cast<float*>(out)[idx] += v;
                     else if (MODE == kAtomicF32) atomicAdd(static_cast<float*>(out) + idx, v);
-                    else static_cast<bf16*>(out)[idx] = static_cast<bf16>(v);
+                    else static_cast<bf16*>(out)[idx] = static_cast<bf16>(stored_value<MODE>(v));
                 }
             }
         }
@@ -900,6 +907,7 @@ static int launch_tile(const bf16* A, const bf16* W, void* out, int M, int N, in
         case kGatedReluBF16: return launch_tile_mode<WMT, WNT, kGatedReluBF16>(A, W, out, M, N, K, 1, blocked, stream);
         case kGatedGeluBF16: return launch_tile_mode<WMT, WNT, kGatedGeluBF16>(A, W, out, M, N, K, 1, blocked, stream);
         case kGatedExtraBF16: return launch_tile_mode<WMT, WNT, kGatedExtraBF16>(A, W, out, M, N, K, 1, blocked, stream);
+        case kSquaredReluBF16: return launch_tile_mode<WMT, WNT, kSquaredReluBF16>(A, W, out, M, N, K, 1, blocked, stream);
         default: return launch_tile_mode<WMT, WNT, kStoreBF16>(A, W, out, M, N, K, 1, blocked, stream);
     }
 }
@@ -920,6 +928,7 @@ static int launch_tile_direct(const bf16* A, const bf16* W, void* out, int M, in
         case kGatedReluBF16: return LLME_DIRECT(kGatedReluBF16);
         case kGatedGeluBF16: return LLME_DIRECT(kGatedGeluBF16);
         case kGatedExtraBF16: return LLME_DIRECT(kGatedExtraBF16);
+        case kSquaredReluBF16: return LLME_DIRECT(kSquaredReluBF16);
         default: return LLME_DIRECT(kStoreBF16);
     }
 #undef LLME_DIRECT
@@ -1011,7 +1020,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const bf16* __rest
             if (MODE == kStoreF32) static_cast<float*>(out)[idx] = s[e];
             else if (MODE == kAddF32) static_cast<float*>(out)[idx] += s[e];
             else if (MODE == kAtomicF32) atomicAdd(static_cast<float*>(out) + idx, s[e]);
-            else static_cast<bf16*>(out)[idx] = static_cast<bf16>(s[e]);
+            else static_cast<bf16*>(out)[idx] = static_cast<bf16>(stored_value<MODE>(s[e]));
         }
     }
 }
@@ -1029,6 +1038,7 @@ static void launch_skinny(const bf16* x, const bf16* w, void* out, int M, int N,
     if (mode == kStoreF32) LLME_SK(kStoreF32);
     else if (mode == kAddF32) LLME_SK(kAddF32);
     else if (mode == kAtomicF32) LLME_SK(kAtomicF32);
+    else if (mode == kSquaredReluBF16) LLME_SK(kSquaredReluBF16);
     else LLME_SK(kStoreBF16);
 #undef LLME_SK
 }
@@ -1047,7 +1057,8 @@ using namespace llme;
 
 // a [M, K], w [N, K] bfloat16; out [M, N] float32 (out_dtype 0) or bfloat16 (1).
 // accumulate (float32 only) adds into out. gated: w holds gate and up rows interleaved in
-// groups of 16 and out is bfloat16 [M, N / 2] = silu(gate) * up (tile kernel only).
+// groups of 16 and out is bfloat16 [M, N / 2] = silu(gate) * up (tile kernel only); gated 5: no gate, out is bfloat16
+// [M, N] = max(product, 0)^2 (both kernels).
 // nw, ksplit: 0 lets the entry point choose the skinny kernel's wavefronts per workgroup and
 // the split over k; tile_shape: 0 chooses, 64 / 128 force the tile kernel with that tile
 // edge also for small M (for tests and measurements), 128096, 128064, 96128, 96064 tiles of 128 x 96 and so on. blocked: w is stored in 1 KB blocks of
@@ -1063,10 +1074,13 @@ extern "C" int llme_gemm_bf16(const void* a, const void* w, void* out, int out_d
     if (K <= 0 || K % 8 != 0 || K >= (1 << 23)) return kErrUnsupported;   // 256 rows of K must stay below 2^32 bytes
     if (out_dtype != kF32 && out_dtype != kBF16) return kErrBadArgument;
     if (accumulate && out_dtype != kF32) return kErrBadArgument;
+    const bool squared = gated == 5;
+    if (squared) gated = 0;
+    if (squared && (out_dtype != kBF16 || accumulate)) return kErrBadArgument;
     if (gated && (out_dtype != kBF16 || N % 32 != 0 || accumulate)) return kErrBadArgument;
     const bf16* A = static_cast<const bf16*>(a);
     const bf16* W = static_cast<const bf16*>(w);
-    int mode = out_dtype == kBF16 ? kStoreBF16 : (accumulate ? kAddF32 : kStoreF32);
+    int mode = squared ? kSquaredReluBF16 : out_dtype == kBF16 ? kStoreBF16 : (accumulate ? kAddF32 : kStoreF32);
     // Up to 16 rows: the skinny kernel (one row tile). 17 to 64 rows: the skinny kernel re-reads
     // the activations from L2 once per 16 output columns, which costs more than the weights
     // themselves, so wide outputs and sums that can be cut over k go to the 64 x 64 tile kernel.
@@ -1118,7 +1132,7 @@ extern "C" int llme_gemm_bf16(const void* a, const void* w, void* out, int out_d
         const long wg128 = static_cast<long>((M + 127) / 128) * ((N + 127) / 128);
         // (a stored output with fewer than 96 tiles of 128 x 128 fills the chip better in 64 x 64 tiles:
         // q/k/v of the 1B sizes at 273 rows 12.6 against 16.0 us; sums that are cut over k keep the larger tiles)
-        const long enough = (mode == kStoreF32 || mode == kStoreBF16) ? 96 : 64;
+        const long enough = (mode == kStoreF32 || is_stored_bf16(mode)) ? 96 : 64;
         tile_shape = (M > 64 && wg128 >= enough) ? 128 : 64;
         if (tile_shape == 128 && wg128 < 4 * cus && !(mode == kAddF32 && wg128 <= cus && K >= 4096)) {
             // Medium outputs: narrower tiles can fill the compute units (two workgroups

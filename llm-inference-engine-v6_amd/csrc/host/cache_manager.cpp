@@ -8,7 +8,9 @@
 //
 // Layers with the same needs form a group with a page pool and block tables of its own: a
 // "full" group keeps every token of a request; a "window" group gives pages back once every
-// position in them lies behind the window of the next token. Beside the pages, every live
+// position in them lies behind the window of the next token; a "chunk" group gives them back
+// once the next token starts or lies in a later chunk (stretches of equal length counted from the
+// sequence's start, a token reading its own chunk only). Beside the pages, every live
 // request holds a slot: a row in each fixed-size state tensor.
 //
 // Plain C++ with a C interface (handles and integer codes), no GPU calls: the Python classes in
@@ -56,11 +58,14 @@ private:
     std::vector<char> held_;
 };
 
+enum GroupKind : int { kFullGroup = 0, kWindowGroup = 1, kChunkGroup = 2 };
+
 struct Group {
-    bool window = false;
-    int window_len = 0;
+    GroupKind kind = kFullGroup;
+    int window_len = 0;                             // tokens of the window, or of a chunk
     PagePool pool;
-    Group(bool w, int wl, int pages) : window(w), window_len(wl), pool(pages) {}
+    Group(GroupKind k, int wl, int pages) : kind(k), window_len(wl), pool(pages) {}
+    bool gives_back() const { return kind != kFullGroup; }          // pages leave in front of the request's end
 };
 
 struct Request {
@@ -76,7 +81,7 @@ public:
     CacheManager(int page_size, int max_requests) : page_size_(page_size), max_requests_(max_requests) {
         for (int s = max_requests - 1; s >= 0; --s) free_slots_.push_back(s);
     }
-    void add_group(bool window, int window_len, int pages) { groups_.emplace_back(window, window_len, pages); }
+    void add_group(GroupKind kind, int window_len, int pages) { groups_.emplace_back(kind, window_len, pages); }
     int num_groups() const { return static_cast<int>(groups_.size()); }
     Group* group(int g) { return g >= 0 && g < num_groups() ? &groups_[static_cast<size_t>(g)] : nullptr; }
     Request* find(int64_t key) {
@@ -102,7 +107,8 @@ public:
 
     // First logical block that a token at `position` reads in this group.
     long first_needed_block(const Group& g, long position) const {
-        if (!g.window) return 0;
+        if (g.kind == kFullGroup) return 0;
+        if (g.kind == kChunkGroup) return position / g.window_len * g.window_len / page_size_;
         const long lo = position - g.window_len + 1;
         return (lo > 0 ? lo : 0) / page_size_;
     }
@@ -114,7 +120,7 @@ public:
         out.clear();
         const long first = first_needed_block(g, r.length);
         const long last = (r.length + n_new - 1) / page_size_;
-        if (!g.window) {                            // the table has no holes: only its end grows
+        if (!g.gives_back()) {                      // the table has no holes: only its end grows
             for (long b = std::max<long>(first, static_cast<long>(table.size())); b <= last; ++b) out.push_back(b);
             return;
         }
@@ -186,8 +192,8 @@ public:
         return 1;
     }
 
-    // The step wrote n_new tokens: the request is that much longer, and window groups give back
-    // the pages no later token will read.
+    // The step wrote n_new tokens: the request is that much longer, and window and chunk groups give
+    // back the pages no later token will read.
     int commit(int64_t key, long n_new) {
         Request* r = find(key);
         if (!r) return LLME_HOST_NOT_LIVE;
@@ -195,7 +201,7 @@ public:
         r->length += n_new;
         for (int gi = 0; gi < num_groups(); ++gi) {
             Group& g = groups_[static_cast<size_t>(gi)];
-            if (!g.window) continue;
+            if (!g.gives_back()) continue;
             std::vector<int>& table = r->tables[static_cast<size_t>(gi)];
             const long keep_from = first_needed_block(g, r->length);       // the next token's first block
             const long end = std::min<long>(keep_from, static_cast<long>(table.size()));
@@ -280,13 +286,14 @@ int llme_pool_free_pages(void* p) { return static_cast<PagePool*>(p)->free_pages
 int llme_pool_is_held(void* p, int page) { return static_cast<PagePool*>(p)->is_held(page) ? 1 : 0; }
 
 // ---- the manager ----
-void* llme_cm_create(int n_groups, const int* is_window, const int* window, const int* num_pages, int page_size,
+// kind per group: 0 full, 1 window, 2 chunk; window: the window's or the chunk's length in tokens
+void* llme_cm_create(int n_groups, const int* kind, const int* window, const int* num_pages, int page_size,
                      int max_requests) {
     if (n_groups < 0 || page_size <= 0 || max_requests <= 0) return nullptr;
     for (int g = 0; g < n_groups; ++g)
-        if (num_pages[g] <= 0 || (is_window[g] && window[g] <= 0)) return nullptr;
+        if (num_pages[g] <= 0 || kind[g] < 0 || kind[g] > 2 || (kind[g] != 0 && window[g] <= 0)) return nullptr;
     CacheManager* m = new CacheManager(page_size, max_requests);
-    for (int g = 0; g < n_groups; ++g) m->add_group(is_window[g] != 0, window[g], num_pages[g]);
+    for (int g = 0; g < n_groups; ++g) m->add_group(static_cast<llme_host::GroupKind>(kind[g]), window[g], num_pages[g]);
     return m;
 }
 void llme_cm_destroy(void* h) { delete static_cast<CacheManager*>(h); }
@@ -377,7 +384,7 @@ int llme_cm_commit_batch(void* h, int S, const int64_t* keys, long n_new) {
 // What a recorded decode step needs before every replay, in one call: for each of the S requests
 // its length (the new token's position) and slot, and into the block tables of every group
 // (rows of `width` entries, group after group) the entries [done, blocks) that are not there
-// yet; window groups are written whole (their early entries turn into -1 over time). The caller
+// yet; window and chunk groups are written whole (their early entries turn into -1 over time). The caller
 // keeps serials[i] and done[g * S + i] between calls (both start at 0): a request in place i
 // that is not the one of the last call (another key, or the same key admitted anew) has its
 // rows written from their start. Returns 0 or an error code.
@@ -397,7 +404,7 @@ int llme_cm_fill_decode(void* h, int S, const int64_t* keys, int width, int* len
             const int nb = static_cast<int>(std::min<size_t>(t.size(), static_cast<size_t>(width)));
             int* row = tables + (static_cast<size_t>(g) * S + i) * width;
             int& d = done[g * S + i];
-            const int lo = (m->group(g)->window || !same) ? 0 : std::min(d, nb);
+            const int lo = (m->group(g)->gives_back() || !same) ? 0 : std::min(d, nb);
             for (int b = lo; b < nb; ++b) row[b] = t[static_cast<size_t>(b)];
             d = nb;
         }
@@ -420,7 +427,7 @@ int llme_cm_lengths(void* h, int S, const int64_t* keys, long* out) {
 // tokens' positions and request indices (T = sum of new_lens values each), the first row of every
 // request (S + 1), the tokens cached before the step (S), the slots (S), and for every group the rows
 // of the block table, `width` entries each (entries behind a request's last page are 0; pages of a
-// window group that were given back stay -1: no token of the step reads them). The arrays are
+// window or chunk group that were given back stay -1: no token of the step reads them). The arrays are
 // written in the caller's one buffer at the given places. Returns the highest position of the
 // step, or an error code (negative).
 long llme_cm_fill_step(void* h, int S, const int64_t* keys, const int* new_lens, int width, int* positions,

@@ -1,5 +1,5 @@
 // A sublayer's result normed before it joins the residual stream ("sandwich" layers):
-//   h[t] += w_post * y[t] / sqrt(mean(y[t]^2) + eps)
+//   h[t] += scale * (w_post * y[t] / sqrt(mean(y[t]^2) + eps))
 // and, in the same pass over the row, the norm in front of the next sublayer:
 //   x[t] = w_next * h[t] / sqrt(mean(h[t]^2) + eps)      (h as just updated)
 // or, where x is asked for without a weight, the updated row as it is in the activation type (x[t] = h[t]: layers
@@ -7,7 +7,7 @@
 // y and h are 32-bit; the weights multiply as given (a norm whose checkpoint stores the distance from one
 // hands over 1 + w). The products are evaluated (w * v) * inv, as the norm kernel evaluates them, so that a
 // row is rounded to the same values whichever kernel norms it. One workgroup a row; the row waits in LDS
-// between the two passes. Also here: a stream scaled by a constant (an embedding's multiplier).
+// between the two passes. Also here: a stream scaled by a constant (an embedding's multiplier) and a soft cap on logits.
 #include "common.h"
 
 namespace llme {
@@ -15,7 +15,7 @@ namespace llme {
 template <typename TW, typename TN, typename TO>
 __global__ __launch_bounds__(256) void norm_add_kernel(const float* __restrict__ y, const TW* __restrict__ w_post,
                                                        float* __restrict__ h, const TN* __restrict__ w_next,
-                                                       TO* __restrict__ x_out, int H, float eps) {
+                                                       TO* __restrict__ x_out, int H, float eps, float scale) {
     extern __shared__ float row[];
     __shared__ float scratch[4];
     const int t = blockIdx.x;
@@ -30,7 +30,7 @@ __global__ __launch_bounds__(256) void norm_add_kernel(const float* __restrict__
     const float inv = 1.0f / sqrtf(block_sum(ss, scratch, 4) / static_cast<float>(H) + eps);
     float ss2 = 0.f;
     for (int i = threadIdx.x; i < H; i += 256) {
-        const float v = hr[i] + (to_float(w_post[i]) * row[i]) * inv;
+        const float v = fmaf(scale, (to_float(w_post[i]) * row[i]) * inv, hr[i]);
         hr[i] = v;
         row[i] = v;
         ss2 = fmaf(v, v, ss2);
@@ -73,7 +73,7 @@ template <> __device__ __forceinline__ void na_store4<bf16>(bf16* p, const float
 template <typename TW, typename TN, typename TO, int NV>
 __global__ __launch_bounds__(256) void norm_add_vec_kernel(const float* __restrict__ y, const TW* __restrict__ w_post,
                                                            float* __restrict__ h, const TN* __restrict__ w_next,
-                                                           TO* __restrict__ x_out, int H, float eps) {
+                                                           TO* __restrict__ x_out, int H, float eps, float scale) {
     __shared__ float scratch[4];
     const int t = blockIdx.x;
     const float* yr = y + static_cast<size_t>(t) * H;
@@ -103,7 +103,7 @@ __global__ __launch_bounds__(256) void norm_add_vec_kernel(const float* __restri
         const int i = (threadIdx.x + 256 * k) * 4;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-            hv[k][e] += (wv[k][e] * yv[k][e]) * inv;
+            hv[k][e] = fmaf(scale, (wv[k][e] * yv[k][e]) * inv, hv[k][e]);
             ss2 = fmaf(hv[k][e], hv[k][e], ss2);
         }
         if (i < H) na_store4(hr + i, hv[k]);
@@ -134,12 +134,18 @@ __global__ void scale_kernel(float* __restrict__ x, size_t n, float s) {
     if (i < n) x[i] *= s;
 }
 
+// x <- cap tanh(x / cap)
+__global__ void soft_cap_kernel(float* __restrict__ x, size_t n, float cap) {
+    const size_t i = static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x;
+    if (i < n) x[i] = cap * tanhf(x[i] / cap);
+}
+
 }  // namespace llme
 
 using namespace llme;
 
 extern "C" int llme_norm_add(const float* y, const void* w_post, int w_dtype, float* h, const void* w_next,
-                             int wn_dtype, void* x_out, int xo_dtype, int T, int H, float eps, hipStream_t stream) {
+                             int wn_dtype, void* x_out, int xo_dtype, int T, int H, float eps, float scale, hipStream_t stream) {
     if (T <= 0) return 0;
     if (H <= 0 || H > 16000) return kErrUnsupported;
     const size_t lds = static_cast<size_t>(H) * sizeof(float);
@@ -149,7 +155,7 @@ extern "C" int llme_norm_add(const float* y, const void* w_post, int w_dtype, fl
     const int nv = !vec ? 0 : H <= 2048 ? 2 : H <= 4096 ? 4 : 8;
 #define LLME_NAV(TW, TN, TO, NV)                                                                          \
     hipLaunchKernelGGL((norm_add_vec_kernel<TW, TN, TO, NV>), dim3(T), dim3(256), 0, stream, y,           \
-                       static_cast<const TW*>(w_post), h, static_cast<const TN*>(w_next), static_cast<TO*>(x_out), H, eps)
+                       static_cast<const TW*>(w_post), h, static_cast<const TN*>(w_next), static_cast<TO*>(x_out), H, eps, scale)
 #define LLME_NA(TW, TN, TO)                                                                               \
     do {                                                                                                  \
         if (nv == 2) LLME_NAV(TW, TN, TO, 2);                                                             \
@@ -158,7 +164,7 @@ extern "C" int llme_norm_add(const float* y, const void* w_post, int w_dtype, fl
         else                                                                                              \
             hipLaunchKernelGGL((norm_add_kernel<TW, TN, TO>), dim3(T), dim3(256), lds, stream, y,         \
                                static_cast<const TW*>(w_post), h, static_cast<const TN*>(w_next),         \
-                               static_cast<TO*>(x_out), H, eps);                                          \
+                               static_cast<TO*>(x_out), H, eps, scale);                                          \
     } while (0)
     if (w_next == nullptr) {
         // nothing more, or the updated rows as they are in x_out's type
@@ -185,6 +191,13 @@ extern "C" int llme_norm_add(const float* y, const void* w_post, int w_dtype, fl
 extern "C" int llme_scale_f32(float* x, size_t n, float s, hipStream_t stream) {
     if (n == 0) return 0;
     hipLaunchKernelGGL(scale_kernel, dim3(static_cast<unsigned>((n + 255) / 256)), dim3(256), 0, stream, x, n, s);
+    return launch_status();
+}
+
+extern "C" int llme_soft_cap_f32(float* x, size_t n, float cap, hipStream_t stream) {
+    if (n == 0) return 0;
+    if (!(cap > 0.f)) return kErrBadArgument;
+    hipLaunchKernelGGL(soft_cap_kernel, dim3(static_cast<unsigned>((n + 255) / 256)), dim3(256), 0, stream, x, n, cap);
     return launch_status();
 }
 

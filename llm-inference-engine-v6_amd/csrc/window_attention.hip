@@ -5,12 +5,15 @@
 //     qh = (head, map) reads key head (head / (heads / nv)) * maps + map and value head head / (heads / nv);
 //   * a score is scale * q . k, then softcap * tanh(score / softcap) where softcap > 0;
 //   * a query at position p sees key j <= p with p - j < window (window 0: every j <= p) or j < keep_first (the first
-//     tokens of a sequence stay visible behind a sliding window, at their true positions);
+//     tokens of a sequence stay visible behind a sliding window, at their true positions); with `chunk` > 0 it sees the
+//     keys j <= p of its own stretch of `chunk` positions, counted from the sequence's start (chunk and window exclude
+//     each other);
 //   * `slopes` (one number a head): a score loses slope_h (p - j), a bias that grows with the distance;
 //   * `sinks` (one number a head): the softmax's denominator also holds e^(sink_h), a key without a value.
 //
 // Three steps: `qk_prepare` turns the input product's 32-bit rows into queries and cache entries (an RMS norm per
-// head with a weight over the head's entries where given, a rotation of the first `rot` entries by position x
+// head with a weight over the head's entries where given, or without one (`unit_norm`; a rotation leaves a head's length
+// as it is, so a norm without a weight is the same in front of it and behind it), a rotation of the first `rot` entries by position x
 // frequency, entry i with entry i + rot / 2 or, `pairs` = 1, entry 2 i with entry 2 i + 1; queries times a temperature
 // 1 + coef ln(floor((p + 1) / every) + 1) where `every` > 0; nk = 0: the layer reads another layer's keys and values
 // and only its queries are made), an attention kernel leaves per run of keys the maximum, the sum and the unscaled weighted values of
@@ -40,7 +43,7 @@ constexpr int kMaxHeadEntries = 256;
 template <typename TQ, typename TC, typename TW>
 __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict__ p, int ld, int nq, int nk, int nv, int dk, int dv,
                                                          int k_col, int v_col, const TW* __restrict__ wq, const TW* __restrict__ wk,
-                                                         float eps, const float* __restrict__ inv_freq, int rot, int pairs,
+                                                         int unit_norm, float eps, const float* __restrict__ inv_freq, int rot, int pairs,
                                                          float qt_coef, int qt_every,
                                                          const int* __restrict__ positions, const int* __restrict__ seq_idx,
                                                          const int* __restrict__ block_table, int max_blocks,
@@ -70,19 +73,19 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict
         const float* hp = row + (is_q ? head * dk : k_col + head * dk);
         const TW* w = is_q ? wq : wk;
         float r = 1.f;
-        if (w != nullptr) {
+        if (w != nullptr || unit_norm) {
             float ss = 0.f;
             for (int e = lane; e < dk; e += 64) ss = fmaf(hp[e], hp[e], ss);
             r = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(dk) + eps);
         }
         for (int e = lane; e < dk; e += 64) {
             const float raw = hp[e];
-            float v = w != nullptr ? raw * r * to_float(w[e]) : raw;
+            float v = w != nullptr ? raw * r * to_float(w[e]) : raw * r;
             if (e < rot) {
                 const bool first = pairs ? (e & 1) == 0 : e < half;
                 const int f = pairs ? e >> 1 : (e < half ? e : e - half);
                 const int pe = pairs ? e ^ 1 : (e < half ? e + half : e - half);
-                const float other = w != nullptr ? hp[pe] * r * to_float(w[pe]) : hp[pe];
+                const float other = w != nullptr ? hp[pe] * r * to_float(w[pe]) : hp[pe] * r;
                 const float sn = sn_t[f], cs = cs_t[f];
                 v = first ? v * cs - other * sn : v * cs + other * sn;
             }
@@ -101,17 +104,13 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict
     }
 }
 
-__device__ __forceinline__ bool key_visible(int key, int pos, int window, int keep_first) {
-    return key <= pos && (window <= 0 || pos - key < window || key < keep_first);
-}
-
 // One workgroup per (token, query head): NW wavefronts take every NW-th chunk of 64 keys and join through LDS.
 template <typename TQ, typename TC, int NW>
 __global__ __launch_bounds__(NW * 64) void window_attention_kernel(
     const TQ* __restrict__ q, const TC* __restrict__ k_cache, const TC* __restrict__ v_cache, float* __restrict__ part_o,
     float* __restrict__ part_ml, const int* __restrict__ positions, const int* __restrict__ seq_idx,
     const int* __restrict__ block_table, int max_blocks, int nq, int nk, int nv, int maps, int dk, int dv, int page, float scale,
-    float softcap, int window, int keep_first, const float* __restrict__ slopes) {
+    float softcap, int window, int keep_first, int chunk, const float* __restrict__ slopes) {
     constexpr int PER_LANE = kMaxHeadEntries / kWave;
     __shared__ float qs[kMaxHeadEntries];
     __shared__ float join_m[NW], join_l[NW];
@@ -124,7 +123,7 @@ __global__ __launch_bounds__(NW * 64) void window_attention_kernel(
     const int pos = positions[t];
     const int* table = block_table + static_cast<size_t>(seq_idx[t]) * max_blocks;
     const int hi = pos + 1;
-    const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    const int lo = chunk > 0 ? pos - pos % chunk : (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
     const int kept = keep_first < lo ? keep_first : lo;        // the first tokens that lie in front of the window
     const float slope = slopes != nullptr ? slopes[head] : 0.f;
 
@@ -336,13 +335,14 @@ __global__ __launch_bounds__(256) void window_attention_finish_kernel(const floa
 using namespace llme;
 
 extern "C" int llme_qk_prepare(const float* p, int ld, int nq, int nk, int nv, int dk, int dv, int k_col, int v_col,
-                               const void* wq, const void* wk, int w_dtype, float eps, const float* inv_freq, int rot,
+                               const void* wq, const void* wk, int w_dtype, int unit_norm, float eps, const float* inv_freq, int rot,
                                int pairs, float qt_coef, int qt_every, const int* positions, const int* seq_idx, const int* block_table, int max_blocks, void* q_out,
                                int q_dtype, void* k_cache, void* v_cache, int cache_dtype, int page, int T, hipStream_t stream) {
     if (T <= 0) return 0;
     if (dk <= 0 || page <= 0 || rot < 0 || rot > dk || rot % 2 != 0 || qt_every < 0) return kErrBadArgument;
     if (nk > 0 && (dv <= 0 || nv <= 0 || nk % nv != 0 || k_cache == nullptr || v_cache == nullptr)) return kErrBadArgument;
     if (nk == 0) nv = 0;                    // (queries only: the keys and values are another layer's)
+    if (unit_norm && (wq != nullptr || wk != nullptr)) return kErrBadArgument;
     if ((nk > 0 && (wq == nullptr) != (wk == nullptr)) || (rot > 0 && inv_freq == nullptr)) return kErrBadArgument;
     if (nk > 0 && v_col < 0 && (nk != nv || dk != dv)) return kErrBadArgument;
     if (dk > kMaxHeadEntries) return kErrBadArgument;
@@ -352,7 +352,7 @@ extern "C" int llme_qk_prepare(const float* p, int ld, int nq, int nk, int nv, i
     const dim3 grid(T, want < head_groups ? (want > 0 ? want : 1) : head_groups);
 #define LLME_PREP(TQ, TC, TW)                                                                                              \
     hipLaunchKernelGGL((qk_prepare_kernel<TQ, TC, TW>), grid, dim3(256), 0, stream, p, ld, nq, nk, nv, dk, dv, k_col, v_col, \
-                       static_cast<const TW*>(wq), static_cast<const TW*>(wk), eps, inv_freq, rot, pairs, qt_coef, qt_every, positions, seq_idx, \
+                       static_cast<const TW*>(wq), static_cast<const TW*>(wk), unit_norm, eps, inv_freq, rot, pairs, qt_coef, qt_every, positions, seq_idx, \
                        block_table, max_blocks, static_cast<TQ*>(q_out), static_cast<TC*>(k_cache), static_cast<TC*>(v_cache), page)
     if (q_dtype != cache_dtype) return kErrBadArgument;
     if (q_dtype == kF32 && w_dtype == kF32) LLME_PREP(float, float, float);
@@ -366,12 +366,12 @@ extern "C" int llme_qk_prepare(const float* p, int ld, int nq, int nk, int nv, i
 extern "C" int llme_window_attention(const void* q, int q_dtype, const void* k_cache, const void* v_cache, int cache_dtype,
                                      float* part_o, float* part_ml, const int* positions, const int* seq_idx,
                                      const int* block_table, int max_blocks, int T, int nq, int nk, int nv, int dk, int dv, int page,
-                                     float scale, float softcap, int window, int keep_first, const float* slopes,
+                                     float scale, float softcap, int window, int keep_first, int chunk, const float* slopes,
                                      hipStream_t stream) {
     if (T <= 0) return 0;
     if (dk <= 0 || dk > kMaxHeadEntries || dv <= 0 || dv > kMaxHeadEntries || nv <= 0 || nk % nv != 0 || page <= 0) return kErrBadArgument;
     const int maps = nk / nv;
-    if (nq % nk != 0 || window < 0 || keep_first < 0) return kErrBadArgument;
+    if (nq % nk != 0 || window < 0 || keep_first < 0 || chunk < 0 || (chunk > 0 && (window > 0 || keep_first > 0))) return kErrBadArgument;
     const dim3 grid(T, nq);
     const bool few = static_cast<long>(T) * nq < 4096;
 #define LLME_WATT(TQ, TC)                                                                                          \
@@ -380,12 +380,12 @@ extern "C" int llme_window_attention(const void* q, int q_dtype, const void* k_c
             hipLaunchKernelGGL((window_attention_kernel<TQ, TC, 8>), grid, dim3(8 * 64), 0, stream,                \
                                static_cast<const TQ*>(q), static_cast<const TC*>(k_cache), static_cast<const TC*>(v_cache), \
                                part_o, part_ml, positions, seq_idx, block_table, max_blocks, nq, nk, nv, maps, dk, dv, page, \
-                               scale, softcap, window, keep_first, slopes);                                              \
+                               scale, softcap, window, keep_first, chunk, slopes);                                              \
         else                                                                                                       \
             hipLaunchKernelGGL((window_attention_kernel<TQ, TC, 1>), grid, dim3(64), 0, stream,                    \
                                static_cast<const TQ*>(q), static_cast<const TC*>(k_cache), static_cast<const TC*>(v_cache), \
                                part_o, part_ml, positions, seq_idx, block_table, max_blocks, nq, nk, nv, maps, dk, dv, page, \
-                               scale, softcap, window, keep_first, slopes);                                              \
+                               scale, softcap, window, keep_first, chunk, slopes);                                              \
     } while (0)
     if (q_dtype == kF32 && cache_dtype == kF32) LLME_WATT(float, float);
     else if (q_dtype == kBF16 && cache_dtype == kBF16) LLME_WATT(bf16, bf16);

@@ -4,8 +4,8 @@
 // A wavefront takes 16 consecutive (token, head) pairs of one request that read the same key head (the heads of a
 // value head fastest, so with 16 heads on a value head a tile is one token, with one head 16 tokens); every row has
 // its own position and so its own visible keys. Keys are walked in blocks of 32: the blocks that hold the first
-// keep_first tokens where they lie in front of the window, then the blocks from the window's start of the tile's
-// first row to the position of its last. The blocks of a tile are cut into `nsplit` runs (grid z); every run leaves
+// keep_first tokens where they lie in front of the window, then the blocks from the window's (or the chunk's) start of the
+// tile's first row to the position of its last. The blocks of a tile are cut into `nsplit` runs (grid z); every run leaves
 // its maximum, sum and unscaled weighted values, which window_attention_finish joins in the order of the runs; where
 // there is one run (prompts) and a head has one map, the kernel can finish its rows itself (sink, a gate per head, a
 // scale) and write them in bfloat16.
@@ -38,7 +38,7 @@ struct WindowArgs {
     const int* positions;
     const int* q_start;
     const int* block_table;
-    int max_blocks, T, nq, nk, nv, maps, per_value_head, dk, dv, page, page_shift, window, keep_first, nsplit;
+    int max_blocks, T, nq, nk, nv, maps, per_value_head, dk, dv, page, page_shift, window, keep_first, chunk, nsplit;
     float scale, softcap;
     const float* slopes;        // [nq / maps] or null: a score loses slope (position - key)
     // Where the keys are in one run and a head has one map, the kernel may finish a row itself instead of leaving its
@@ -50,6 +50,12 @@ struct WindowArgs {
     int ld_out, ld_gate;
     float out_scale;
 };
+
+// The first key of the stretch that a query at `pos` sees: its window's start, its chunk's, or the sequence's.
+__device__ __forceinline__ int first_seen(const WindowArgs& a, int pos) {
+    if (a.chunk > 0) return pos - pos % a.chunk;
+    return (a.window > 0 && pos - a.window + 1 > 0) ? pos - a.window + 1 : 0;
+}
 
 // The end of a tile's walk: the row's parts into part_o / part_ml, or (a.out given) the finished row. l is the row's
 // whole sum already.
@@ -104,7 +110,7 @@ __device__ __forceinline__ float capped_score(float s, float k, float cap) {
 // beyond the request), or a key lies behind the tile's last; otherwise every weight counts and no test is made.
 template <int NVM, bool EDGE, int CAP>
 __device__ __forceinline__ void window_block(const WindowArgs& a, const f32x4 (&sc)[2], bf16x8 (&vf)[NVM], f32x4 (&acc)[NVM], float& m,
-                                             float& l, int nvt, int key0, int qd, int pos, int pos_max, bool valid, float inv_cap, float slope) {
+                                             float& l, int nvt, int key0, int qd, int pos, int lo, int pos_max, bool valid, float inv_cap, float slope) {
     float p[8];
     float mx = -INFINITY;
 #pragma unroll
@@ -114,7 +120,7 @@ __device__ __forceinline__ void window_block(const WindowArgs& a, const f32x4 (&
         if (CAP == kScoreDistance) v = fmaf(slope, static_cast<float>(key0 + qd * 8 + j - pos), v);
         if (EDGE) {
             const int key = key0 + qd * 8 + j;
-            const bool seen = valid && key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
+            const bool seen = valid && key <= pos && (key >= lo || key < a.keep_first);
             v = seen ? v : -INFINITY;
         }
         p[j] = v;
@@ -199,7 +205,7 @@ __global__ __launch_bounds__(256, (DSM <= 2 && NVM <= 4) ? 4 : NVM <= 4 ? 3 : 2)
     }
 
     // the tile's blocks of 32 keys: [0, nb_kept) and [first_blk, last_blk]
-    const int lo_min = (a.window > 0 && pos_min - a.window + 1 > 0) ? pos_min - a.window + 1 : 0;
+    const int lo = first_seen(a, pos), lo_min = first_seen(a, pos_min), lo_max = first_seen(a, pos_max);
     int first_blk = lo_min >> 5;
     const int last_blk = pos_max >> 5;
     int nb_kept = 0;
@@ -268,9 +274,9 @@ __global__ __launch_bounds__(256, (DSM <= 2 && NVM <= 4) ? 4 : NVM <= 4 ? 3 : 2)
         if (b + 1 < b_end) load_keys(b + 1);                    // the next block's keys travel while this one's weights are made
         // every row sees every key of the block: behind the window's start of the tile's last row, up to the tile's
         // first position, not among the kept blocks (whose keys may lie beyond keep_first)
-        const bool inner = all_valid && b >= nb_kept && key0 + 31 <= pos_min && (a.window <= 0 || pos_max - key0 < a.window);
-        if (inner) window_block<NVM, false, CAP>(a, sc, vf, acc, m, l, nvt, key0, qd, pos, pos_max, valid, inv_cap, slope);
-        else window_block<NVM, true, CAP>(a, sc, vf, acc, m, l, nvt, key0, qd, pos, pos_max, valid, inv_cap, slope);
+        const bool inner = all_valid && b >= nb_kept && key0 + 31 <= pos_min && key0 >= lo_max;
+        if (inner) window_block<NVM, false, CAP>(a, sc, vf, acc, m, l, nvt, key0, qd, pos, lo, pos_max, valid, inv_cap, slope);
+        else window_block<NVM, true, CAP>(a, sc, vf, acc, m, l, nvt, key0, qd, pos, lo, pos_max, valid, inv_cap, slope);
     }
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
@@ -291,7 +297,7 @@ __global__ __launch_bounds__(256, (DSM <= 2 && NVM <= 4) ? 4 : NVM <= 4 ? 3 : 2)
 // order.
 template <int NVM, bool EDGE, int CAP>
 __device__ __forceinline__ void shared_block(const WindowArgs& a, const f32x4 (&sc)[2], const bf16* lds_v, f32x4 (&acc)[NVM], float& m,
-                                             float& l, int nvt, int key0, int r, int qd, int pos, bool valid, float inv_cap, float slope) {
+                                             float& l, int nvt, int key0, int r, int qd, int pos, int lo, bool valid, float inv_cap, float slope) {
     float p[8];
     float mx = -INFINITY;
 #pragma unroll
@@ -301,7 +307,7 @@ __device__ __forceinline__ void shared_block(const WindowArgs& a, const f32x4 (&
         if (CAP == kScoreDistance) v = fmaf(slope, static_cast<float>(key0 + qd * 8 + j - pos), v);
         if (EDGE) {
             const int key = key0 + qd * 8 + j;
-            const bool seen = valid && key <= pos && (a.window <= 0 || pos - key < a.window || key < a.keep_first);
+            const bool seen = valid && key <= pos && (key >= lo || key < a.keep_first);
             v = seen ? v : -INFINITY;
         }
         p[j] = v;
@@ -388,7 +394,8 @@ __global__ __launch_bounds__(256, 4) void window_attention_mfma_shared_kernel(Wi
     }
 
     // the workgroup's blocks of 32 keys: [0, nb_kept) and [first_blk, last_blk]
-    const int lo_min = (a.window > 0 && wg_pos_min - a.window + 1 > 0) ? wg_pos_min - a.window + 1 : 0;
+    const int lo = first_seen(a, pos), lo_max = first_seen(a, pos_max), tile_lo_min = first_seen(a, pos_min);
+    const int lo_min = first_seen(a, wg_pos_min);
     int first_blk = lo_min >> 5;
     const int last_blk = wg_pos_max >> 5;
     int nb_kept = 0;
@@ -473,7 +480,7 @@ __global__ __launch_bounds__(256, 4) void window_attention_mfma_shared_kernel(Wi
         // (a block behind this tile's last key, or in front of the window's start of its first row and not among the
         // kept ones, has no key for it)
         const bool mine = active && key0 <= pos_max
-                          && (a.window <= 0 || b < nb_kept || key0 + 31 >= pos_min - a.window + 1 || key0 < a.keep_first);
+                          && (b < nb_kept || key0 + 31 >= tile_lo_min || key0 < a.keep_first);
         if (mine) {
             const bf16* lk = lds + buf * (K_ELEMS + V_ELEMS);
             f32x4 sc[2];
@@ -492,9 +499,9 @@ __global__ __launch_bounds__(256, 4) void window_attention_mfma_shared_kernel(Wi
                     }
                 }
             }
-            const bool inner = all_valid && b >= nb_kept && key0 + 31 <= pos_min && (a.window <= 0 || pos_max - key0 < a.window);
-            if (inner) shared_block<NVM, false, CAP>(a, sc, lk + K_ELEMS, acc, m, l, nvt, key0, r, qd, pos, valid, inv_cap, slope);
-            else shared_block<NVM, true, CAP>(a, sc, lk + K_ELEMS, acc, m, l, nvt, key0, r, qd, pos, valid, inv_cap, slope);
+            const bool inner = all_valid && b >= nb_kept && key0 + 31 <= pos_min && key0 >= lo_max;
+            if (inner) shared_block<NVM, false, CAP>(a, sc, lk + K_ELEMS, acc, m, l, nvt, key0, r, qd, pos, lo, valid, inv_cap, slope);
+            else shared_block<NVM, true, CAP>(a, sc, lk + K_ELEMS, acc, m, l, nvt, key0, r, qd, pos, lo, valid, inv_cap, slope);
         }
         if (b + 1 < b_end) stage(buf ^ 1);
         __syncthreads();
@@ -515,11 +522,12 @@ using namespace llme;
 extern "C" int llme_window_attention_mfma(const void* q, const void* k_cache, const void* v_cache, float* part_o, float* part_ml,
                                           const int* positions, const int* q_start, const int* block_table, int max_blocks, int T,
                                           int S, int max_new, int nq, int nk, int nv, int dk, int dv, int page, float scale,
-                                          float softcap, int window, int keep_first, int nsplit, int staged, const float* slopes,
+                                          float softcap, int window, int keep_first, int chunk, int nsplit, int staged, const float* slopes,
                                           void* out, int ld_out, const float* sinks, const float* head_gate, int ld_gate,
                                           float out_scale, hipStream_t stream) {
     if (T <= 0 || S <= 0) return 0;
     if (nv <= 0 || nk % nv != 0 || nq % nk != 0 || max_new <= 0 || nsplit <= 0 || window < 0 || keep_first < 0) return kErrBadArgument;
+    if (chunk < 0 || (chunk > 0 && (window > 0 || keep_first > 0))) return kErrBadArgument;
     if (dk % 8 != 0 || dk > 128 || dv % 16 != 0 || dv > 128 || page % 16 != 0 || (page & (page - 1)) != 0) return kErrUnsupported;
     if (softcap > 0.f && slopes != nullptr) return kErrUnsupported;         // (capped and biased scores: the plain kernel)
     // (finished rows: one run of keys, one map a head, rows of whole 8-byte pieces)
@@ -553,6 +561,7 @@ extern "C" int llme_window_attention_mfma(const void* q, const void* k_cache, co
     a.page_shift = __builtin_ctz(page);
     a.window = window;
     a.keep_first = keep_first;
+    a.chunk = chunk;
     a.nsplit = nsplit;
     a.scale = scale;
     a.softcap = softcap;

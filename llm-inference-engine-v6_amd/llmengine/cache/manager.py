@@ -9,8 +9,9 @@ step never fails for capacity half-way.
 
 Layers with the same needs form a group with a page pool and block tables of its
 own: a "full" group keeps every token of a request; a "window" group gives pages
-back once every position in them lies behind the window of the next token. Beside
-the pages, every live request holds a slot: a row in each fixed-size state tensor.
+back once every position in them lies behind the window of the next token; a "chunk"
+group once the next token belongs to a later chunk (stretches of `window` tokens counted
+from the sequence's start, a token reading its own chunk only). Beside the pages, every live request holds a slot: a row in each fixed-size state tensor.
 
 The bookkeeping itself is C++ (csrc/host/cache_manager.cpp); the classes here name
 groups and requests (any hashable; the C++ side knows them by 64-bit keys) and turn
@@ -63,11 +64,12 @@ class PagePool:
 @dataclass(frozen=True)
 class GroupSpec:
     name: str
-    kind: str = "full"          # "full" | "window"
-    window: int = 0
+    kind: str = "full"          # "full" | "window" | "chunk"
+    window: int = 0             # tokens of the window or of a chunk
     num_pages: int = 0
 
 
+GROUP_KINDS = {"full": 0, "window": 1, "chunk": 2}
 _TEXT_KEYS = 1 << 62            # keys of requests that are not named by a small integer
 
 
@@ -81,10 +83,10 @@ class CacheManager:
         if len(set(names)) != len(names):
             raise ValueError(f"cache groups must have distinct names, got {names}")
         for g in groups:
-            if g.kind not in ("full", "window"):
-                raise ValueError(f"group {g.name}: kind {g.kind!r} is not 'full' or 'window'")
-            if g.kind == "window" and g.window <= 0:
-                raise ValueError(f"group {g.name}: a window group needs window > 0")
+            if g.kind not in GROUP_KINDS:
+                raise ValueError(f"group {g.name}: kind {g.kind!r} is not 'full', 'window' or 'chunk'")
+            if g.kind != "full" and g.window <= 0:
+                raise ValueError(f"group {g.name}: a {g.kind} group needs window > 0")
             if g.num_pages <= 0:
                 raise ValueError("a page pool needs at least one page")
         self.page_size = int(page_size)
@@ -94,7 +96,7 @@ class CacheManager:
         self._lib = native.library()
         n = len(groups)
         arr = ctypes.c_int * max(n, 1)
-        self._h = self._lib.llme_cm_create(n, arr(*[int(g.kind == "window") for g in groups]),
+        self._h = self._lib.llme_cm_create(n, arr(*[GROUP_KINDS[g.kind] for g in groups]),
                                            arr(*[int(g.window) for g in groups]),
                                            arr(*[int(g.num_pages) for g in groups]), self.page_size, self.max_requests)
         if not self._h:
@@ -204,7 +206,7 @@ class CacheManager:
 
     def commit(self, request_id, n_new: int) -> None:
         """The step wrote n_new tokens: the request is that much longer, and window
-        groups give back the pages no later token will read."""
+        and chunk groups give back the pages no later token will read."""
         rc = self._lib.llme_cm_commit(self._h, self._key(request_id), int(n_new))
         if rc == native.NOT_RESERVED:
             raise CacheError(f"request {request_id!r}: commit of {n_new} tokens beyond the reserved pages")

@@ -14,7 +14,7 @@ from .manager import GroupSpec
 
 def group_name(spec: CacheSpec) -> str:
     kind, window = spec.group_key
-    return "full" if kind == "full" else f"window{window}"
+    return "full" if kind == "full" else f"{kind}{window}"
 
 
 def plan_groups(specs: dict[int, CacheSpec | None], num_pages: int | dict[str, int]) -> list[GroupSpec]:

@@ -4,5 +4,6 @@ from . import rilonex  # registers "Rilonex"
 from . import bidirax  # registers "Bidirax"
 from . import zetonex  # registers "Zetonex"
 from . import zapolorn  # registers "Zapolorn"
+from . import lukupel  # registers "Lukupel"
 
-__all__ = ["DecoderModel", "LayerCall", "llama", "rilonex", "bidirax", "zetonex", "zapolorn"]
+__all__ = ["DecoderModel", "LayerCall", "llama", "rilonex", "bidirax", "zetonex", "zapolorn", "lukupel"]

@@ -34,12 +34,17 @@ class DecoderModel(Part):
 
     def __init__(self, config, embedding: TokenEmbedding, layers: list[Block], final_norm: Norm,
                  head: Head, schedule: list[LayerCall] | None = None, names: dict | None = None, streams: int = 0,
-                 pass_input: Part | None = None):
+                 pass_input: Part | None = None, layer_numbers: list[int] | None = None):
         self.config = config
         # streams > 0: the residual is kept as that many streams [streams, T, H] (blocks that know how read and
         # write them); every stream starts as the embedding, and the final norm reads their sum
         self.streams = int(streams)
         self.embedding, self.layers, self.final_norm, self.head = embedding, list(layers), final_norm, head
+        # the numbers under which a checkpoint stores the layers' tensors (a layer without tensors of its own, which
+        # runs on another's with a cache of its own, is a second call in the schedule and not a layer here)
+        self.layer_numbers = list(layer_numbers) if layer_numbers is not None else list(range(len(self.layers)))
+        if len(self.layer_numbers) != len(self.layers) or len(set(self.layer_numbers)) != len(self.layers):
+            raise ValueError(f"{len(self.layers)} layers need as many different numbers, got {self.layer_numbers}")
         self.schedule = list(schedule) if schedule is not None else [LayerCall(i) for i in range(len(layers))]
         # what runs in front of the calls marked `enter`: forward(h, h0, step) replaces the stream h, given the
         # embedding's output h0 (a stack of layers that runs several passes over the same weights)
@@ -58,7 +63,7 @@ class DecoderModel(Part):
     def children(self):
         n = self.names
         out: dict[str, Part] = {n["embedding"]: self.embedding}
-        for i, layer in enumerate(self.layers):
+        for i, layer in zip(self.layer_numbers, self.layers):
             # ("model.layers" names layer 3 "model.layers.3"; a pattern with "{}" puts the number where it says)
             out[n["layers"].format(i) if "{}" in n["layers"] else f"{n['layers']}.{i}"] = layer
         out[n["final_norm"]] = self.final_norm

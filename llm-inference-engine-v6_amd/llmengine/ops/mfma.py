@@ -80,6 +80,32 @@ def gemm_gated(x: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tensor, grou
         gated_activation(gu, out, group, activation)
 
 
+declare("llme_squared_relu", [_vp, _vp, _i, ctypes.c_size_t, _vp])
+
+
+def gemm_squared_relu(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, scratch, choices: KernelChoices | None = None) -> None:
+    """out [T, N] = max(x w^T, 0)^2: in the product's epilogue where the MFMA kernels take the operands; otherwise the
+    product into a 32-bit scratch [T, N] (scratch(shape, dtype) provides it) and the activation kernel."""
+    T, N = out.shape
+    require(out, "out", (torch.float32, torch.bfloat16))
+    if ((choices or DEFAULT).fast_gemm and out.dtype == torch.bfloat16 and N % 8 == 0
+            and gemm_bf16_supported(x, w, out, False)):
+        require(x, "x", torch.bfloat16, (T, None))
+        K = x.shape[1]
+        n_rows, _ = kernels._require_weight(w, "w", torch.bfloat16, K)
+        if n_rows != N:
+            raise kernels.KernelError(f"gemm_squared_relu: {n_rows} weight rows for {N} columns")
+        r = tail_rows(T, choices)
+        for a, b in ((0, T - r), (T - r, T)):
+            if a < b:
+                check(entry("llme_gemm_bf16")(ptr(x[a:b]), ptr(w), ptr(out[a:b]), 1, b - a, N, K, 0, 5, 0, 0, 0,
+                                              1 if kernels.is_blocked(w) else 0, -1, stream()), "gemm_squared_relu")
+        return
+    p = scratch((T, N), torch.float32)
+    kernels.gemm(x, w, p, choices=choices)
+    check(entry("llme_squared_relu")(ptr(p), ptr(out), 0 if out.dtype == torch.float32 else 1, p.numel(), stream()), "squared_relu")
+
+
 declare("llme_gemm_bf16_gated_extra", [_vp, _vp, _vp, _i, _i, _i, _vp, _f, _f, _i, _i, _i, _vp])
 GATED_EXTRA_MIN_ROWS = 17       # fewer rows (decoded tokens) go through the skinny product and the activation kernel
 

@@ -16,9 +16,9 @@ WINDOW_ATTENTION_MAX_ENTRIES = 256          # entries of a key or value head tha
 FINISH_MODES = {"plain": 0, "gate": 1, "difference": 2, "head_gate": 3}
 BIAS_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "swish_clamped": 3}
 
-declare("llme_qk_prepare", [_vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _i, _f, _vp, _i, _i, _f, _i, _vp, _vp, _vp, _i, _vp, _i, _vp,
+declare("llme_qk_prepare", [_vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _i, _i, _f, _vp, _i, _i, _f, _i, _vp, _vp, _vp, _i, _vp, _i, _vp,
                             _vp, _i, _i, _i, _vp])
-declare("llme_window_attention", [_vp, _i, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i, _vp,
+declare("llme_window_attention", [_vp, _i, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i, _i, _vp,
                                   _vp])
 declare("llme_window_attention_finish", [_vp, _vp, _i, _i, _i, _i, _i, _i, _vp, _i, _f, _f, _f, _vp, _vp, _i, _i, _vp])
 declare("llme_gated_bias_act", [_vp, _i, _vp, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _vp, _vp, _vp])
@@ -37,11 +37,11 @@ def _columns(p: torch.Tensor, name: str) -> int:
 def qk_prepare(p: torch.Tensor, step, block_table: torch.Tensor | None, q_out: torch.Tensor, k_cache: torch.Tensor | None,
                v_cache: torch.Tensor | None, nq: int, k_col: int, v_col: int | None, inv_freq: torch.Tensor | None, rot: int,
                wq: torch.Tensor | None = None, wk: torch.Tensor | None = None, eps: float = 0.0, pairs: str = "halves",
-               q_temp: tuple[float, int] | None = None, dk: int | None = None) -> None:
+               q_temp: tuple[float, int] | None = None, dk: int | None = None, unit_norm: bool = False) -> None:
     """Rows p [T, ..] (32-bit: nq query heads of dk entries at column 0, the key heads at k_col, the value heads at
     v_col; v_col None: a value head is the key head as projected) -> q_out [T, nq dk] and the cache entries of the
     rows' tokens: k_cache [pages, nk, page, dk], v_cache [pages, nv, dv, page]. wq, wk [dk]: every query and key
-    head is divided by its root mean square (eps inside the root) and multiplied by the weight first. Then the first
+    head is divided by its root mean square (eps inside the root) and multiplied by the weight first; unit_norm: the same without a weight. Then the first
     `rot` entries of a query or key head turn by position * inv_freq[i]: entry i with entry i + rot / 2 (pairs
     "halves") or entry 2 i with entry 2 i + 1 ("neighbours"). q_temp (coef, every): the queries of position p times
     1 + coef ln(floor((p + 1) / every) + 1). k_cache None: only the queries are made (the keys and values are another
@@ -69,6 +69,8 @@ def qk_prepare(p: torch.Tensor, step, block_table: torch.Tensor | None, q_out: t
     need = max(nq * dk, (k_col + nk * dk) if nk else 0, (v_col + nv * dv) if v_col is not None else 0)
     if p.shape[1] < need:
         raise KernelError(f"qk_prepare: rows of {p.shape[1]} columns hold no {need}")
+    if unit_norm and (wq is not None or wk is not None):
+        raise KernelError("qk_prepare: a norm without a weight takes none")
     if rot:
         require(inv_freq, "inv_freq", torch.float32, (rot // 2,))
     if wq is not None:
@@ -79,14 +81,14 @@ def qk_prepare(p: torch.Tensor, step, block_table: torch.Tensor | None, q_out: t
     if q_temp and every <= 0:
         raise KernelError("qk_prepare: the queries' temperature steps every > 0 positions")
     check(entry("llme_qk_prepare")(ptr(p), ld, nq, nk, nv, dk, dv, int(k_col), -1 if v_col is None else int(v_col), ptr(wq), ptr(wk),
-                                   code(wq.dtype) if wq is not None else 0, float(eps), ptr(inv_freq) if rot else None, int(rot),
+                                   code(wq.dtype) if wq is not None else 0, 1 if unit_norm else 0, float(eps), ptr(inv_freq) if rot else None, int(rot),
                                    1 if pairs == "neighbours" else 0, coef, every,
                                    ptr(step.positions), ptr(step.seq_idx), ptr(block_table) if nk else None,
                                    block_table.shape[1] if nk else 0, ptr(q_out), code(q_out.dtype), ptr(k_cache), ptr(v_cache),
                                    code(q_out.dtype), page, T, stream()), "qk_prepare")
 
 
-declare("llme_window_attention_mfma", [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i,
+declare("llme_window_attention_mfma", [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i, _i,
                                        _i, _i, _vp, _vp, _i, _vp, _vp, _i, _f, _vp])
 WINDOW_MFMA_FINISHES = True         # a step whose keys are in one run has its rows finished by the attention kernel (False: tests)
 WINDOW_MFMA_STAGED = True           # prompts' blocks of keys staged once a workgroup through LDS (False: measurements, tests)
@@ -104,7 +106,7 @@ def window_mfma_fits(k_cache: torch.Tensor, v_cache: torch.Tensor, choices=None)
             and max(dk, dv) <= WINDOW_MFMA_MAX_ENTRIES and page % 16 == 0)
 
 
-def window_runs(step, rows_per_token: int, key_heads: int, window: int, keep_first: int) -> tuple[int, int]:
+def window_runs(step, rows_per_token: int, key_heads: int, window: int, keep_first: int, chunk: int = 0) -> tuple[int, int]:
     """(the most tokens a request brings, runs to cut a tile's keys into) for the matrix-core kernel: enough wavefronts
     for four a compute unit, a run no shorter than a block of 32 keys. A step of single tokens plans for requests of
     up to step.plan_len keys where that is set (the step may be recorded and replayed for longer requests)."""
@@ -117,6 +119,8 @@ def window_runs(step, rows_per_token: int, key_heads: int, window: int, keep_fir
         keys = max(c + n for c, n in zip(step.ctx_lens, step.new_lens))
     if window:
         keys = min(keys, window + (16 + rows_per_token - 1) // rows_per_token + min(keep_first, keys))
+    if chunk:
+        keys = min(keys, chunk + (16 + rows_per_token - 1) // rows_per_token)
     tiles = sum((n * rows_per_token + 15) // 16 for n in step.new_lens) * key_heads
     blocks = (keys + 31) // 32 + 1
     runs = max(1, min(WINDOW_MFMA_MAX_RUNS, (4 * mfma.compute_units()) // max(tiles, 1), blocks))
@@ -126,14 +130,14 @@ def window_runs(step, rows_per_token: int, key_heads: int, window: int, keep_fir
     return max_new, runs
 
 
-def _fast_window_attention(q, k_cache, v_cache, step, block_table, nq, scale, softcap, window, keep_first, slopes=None, finish=None):
+def _fast_window_attention(q, k_cache, v_cache, step, block_table, nq, scale, softcap, window, keep_first, slopes=None, finish=None, chunk=0):
     from .choices import choices_of
     if not window_mfma_fits(k_cache, v_cache, choices_of(step)) or (softcap > 0 and slopes is not None):
         return None
     T = q.shape[0]
     _, nk, page, dk = k_cache.shape
     nv, dv = v_cache.shape[1], v_cache.shape[2]
-    max_new, runs = window_runs(step, nq // nk, nk, window, keep_first)
+    max_new, runs = window_runs(step, nq // nk, nk, window, keep_first, chunk)
     out = gate = sinks = None
     ld_out = ld_gate = 0
     out_scale = 1.0
@@ -157,7 +161,7 @@ def _fast_window_attention(q, k_cache, v_cache, step, block_table, nq, scale, so
         part_o = part_ml = None
     check(entry("llme_window_attention_mfma")(ptr(q), ptr(k_cache), ptr(v_cache), ptr(part_o), ptr(part_ml), ptr(step.positions),
                                               ptr(step.q_start), ptr(block_table), block_table.shape[1], T, step.num_seqs, max_new,
-                                              nq, nk, nv, dk, dv, page, float(scale), float(softcap), int(window), int(keep_first),
+                                              nq, nk, nv, dk, dv, page, float(scale), float(softcap), int(window), int(keep_first), int(chunk),
                                               runs, 1 if WINDOW_MFMA_STAGED else 0, ptr(slopes), ptr(out), ld_out, ptr(sinks),
                                               ptr(gate), ld_gate, out_scale, stream()),
           "window_attention_mfma")
@@ -166,8 +170,9 @@ def _fast_window_attention(q, k_cache, v_cache, step, block_table, nq, scale, so
 
 def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, step, block_table: torch.Tensor, nq: int,
                      scale: float, softcap: float = 0.0, window: int = 0, keep_first: int = 0,
-                     slopes: torch.Tensor | None = None, finish: dict | None = None):
-    """Every (token, query head) of the step over the keys of its request that it may see; slopes [heads] (32-bit): the
+                     slopes: torch.Tensor | None = None, finish: dict | None = None, chunk: int = 0):
+    """Every (token, query head) of the step over the keys of its request that it may see (chunk > 0: those of its own
+    stretch of `chunk` positions counted from the sequence's start; not together with a window); slopes [heads] (32-bit): the
     score of head h loses slopes[h] times the distance between query and key. finish: what `window_attention_finish`
     would be asked to do with the parts (out, mode, gate, sinks, out_scale); where the matrix-core kernel walks a
     row's keys in one run it does that itself and "finished" is returned instead of the parts. Returns (part_o
@@ -186,8 +191,10 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         raise KernelError(f"window attention: heads of {dk} and {dv} entries are beyond the kernels' {WINDOW_ATTENTION_MAX_ENTRIES}")
     if slopes is not None:
         require(slopes, "slopes", torch.float32, (nq // (nk // nv),))
+    if chunk and (window or keep_first):
+        raise KernelError("window attention: chunks and a window exclude each other")
     if _fast_window_attention is not None:
-        parts = _fast_window_attention(q, k_cache, v_cache, step, block_table, nq, scale, softcap, window, keep_first, slopes, finish)
+        parts = _fast_window_attention(q, k_cache, v_cache, step, block_table, nq, scale, softcap, window, keep_first, slopes, finish, chunk)
         if parts is not None:
             return parts
     part_o = step.buffer("window_attention.part_o", (1, T, nq, dv), torch.float32)
@@ -195,7 +202,7 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     check(entry("llme_window_attention")(ptr(q), code(q.dtype), ptr(k_cache), ptr(v_cache), code(k_cache.dtype), ptr(part_o),
                                          ptr(part_ml), ptr(step.positions), ptr(step.seq_idx), ptr(block_table),
                                          block_table.shape[1], T, nq, nk, nv, dk, dv, page, float(scale), float(softcap),
-                                         int(window), int(keep_first), ptr(slopes), stream()), "window_attention")
+                                         int(window), int(keep_first), int(chunk), ptr(slopes), stream()), "window_attention")
     return part_o, part_ml
 
 

@@ -4,7 +4,7 @@ from .registry import LayerSpec, PartChoice, build_layer, make_part, register_pa
 from .norm import CenteredRMSNorm, RMSNorm
 from .rope import RotaryEmbedding, inverse_frequencies
 from .embedding import Embedding, OutputHead
-from .mlp import GatedMLP
+from .mlp import GatedMLP, SquaredReluMLP
 from .attention import Attention
 from .block import OutputNormBlock, ParallelBlock, PreNormBlock, SandwichBlock
 from .projected import ParallelMixer, ProjectedMixer
@@ -16,6 +16,7 @@ from .latent_attention import LatentAttention
 from .moe import MixtureOfExperts
 from .window_attention import WindowAttention
 from .linear_attention import GatedLinearAttention
+from .mlstm import MatrixMemory
 from .reentry import PassInput
 
 __all__ = ["PAGE", "Block", "CacheSpec", "FeedForward", "LayerCache", "Mixer", "Norm", "ParamSpec", "Part",
@@ -23,4 +24,4 @@ __all__ = ["PAGE", "Block", "CacheSpec", "FeedForward", "LayerCache", "Mixer", "
            "register_part", "registered", "RMSNorm", "RotaryEmbedding", "inverse_frequencies", "Embedding",
            "OutputHead", "GatedMLP", "Attention", "PreNormBlock", "ParallelMixer", "ProjectedMixer", "RGLRU", "GatedDeltaRule",
            "SigmoidAttention", "HyperConnectionBlock", "CenteredRMSNorm", "SandwichBlock", "LatentAttention",
-           "MixtureOfExperts", "WindowAttention", "PassInput", "ParallelBlock", "OutputNormBlock", "GatedLinearAttention"]
+           "MixtureOfExperts", "WindowAttention", "PassInput", "ParallelBlock", "OutputNormBlock", "GatedLinearAttention", "MatrixMemory", "SquaredReluMLP"]

@@ -173,7 +173,9 @@ class CacheSpec:
            the model's activation type. Layers with the same (kind, window) share a
            page pool and a block table (one page id covers all of them).
     kind:  "full": every token of the request stays; "window": only the last
-           `window` tokens are ever read, pages behind them are given back.
+           `window` tokens are ever read, pages behind them are given back; "chunk": a token
+           reads only its own stretch of `window` tokens, counted from the sequence's start,
+           pages of earlier stretches are given back.
     state: tensors of fixed size per request: name -> (shape, dtype), kept in the
            request's slot, zero when the request is admitted.
     """
@@ -183,10 +185,10 @@ class CacheSpec:
     state: Mapping[str, tuple[tuple[int, ...], torch.dtype]] = field(default_factory=dict)
 
     def __post_init__(self):
-        if self.kind not in ("full", "window"):
-            raise ValueError(f"cache kind {self.kind!r} is not 'full' or 'window'")
-        if self.kind == "window" and self.window <= 0:
-            raise ValueError("a window cache needs window > 0")
+        if self.kind not in ("full", "window", "chunk"):
+            raise ValueError(f"cache kind {self.kind!r} is not 'full', 'window' or 'chunk'")
+        if self.kind != "full" and self.window <= 0:
+            raise ValueError(f"a {self.kind} cache needs window > 0")
 
     def paged_tensors(self, default_dtype: torch.dtype) -> dict[str, tuple[tuple[int, ...], torch.dtype]]:
         """name -> (shape of one page, dtype), the model's activation type where none is given."""
@@ -200,7 +202,7 @@ class CacheSpec:
 
     @property
     def group_key(self) -> tuple:
-        return (self.kind, self.window if self.kind == "window" else 0)
+        return (self.kind, self.window if self.kind != "full" else 0)
 
 
 @dataclass

@@ -140,16 +140,18 @@ class ParallelBlock(Block):
 
 
 class OutputNormBlock(Block):
-    """Norms behind the sublayers only: h += norm1(mixer(h)); h += norm2(ffn(h)). The sublayers read the stream itself
+    """Norms behind the sublayers only: h += c norm1(mixer(h)); h += c norm2(ffn(h)) with a constant c (`residual_scale`, 1
+    unless given). The sublayers read the stream itself
     (rounded to the activation type where that is not 32-bit); a sublayer's result is a 32-bit buffer of its own, and
     the norm behind it, the sum into the stream and the copy of the updated rows that the next sublayer reads (this
     block's feed-forward, or the mixer of the block behind) are one kernel."""
     graph_safe = True
 
     def __init__(self, mixer: Mixer, feed_forward: FeedForward | None, mixer_norm: Norm, ffn_norm: Norm | None,
-                 names: dict | None = None):
+                 names: dict | None = None, residual_scale: float = 1.0):
         self.mixer, self.feed_forward = mixer, feed_forward
         self.mixer_norm, self.ffn_norm = mixer_norm, ffn_norm
+        self.residual_scale = float(residual_scale)
         self.names = {"mixer_norm": "norm1", "mixer": "mix", "ffn_norm": "norm2", "feed_forward": "mlp"}
         if names:
             self.names.update(names)
@@ -163,13 +165,12 @@ class OutputNormBlock(Block):
             out.update({n["ffn_norm"]: self.ffn_norm, n["feed_forward"]: self.feed_forward})
         return out
 
-    @staticmethod
-    def _join(y, post: Norm, h, x) -> None:
-        """h += post(y), and x = the updated rows where x is another buffer than the stream."""
+    def _join(self, y, post: Norm, h, x) -> None:
+        """h += c post(y), and x = the updated rows where x is another buffer than the stream."""
         rms = post.fused_rms()
         if rms is None:
             raise NotImplementedError("output-norm blocks take norms of the plain RMS formula behind their sublayers")
-        ops.norm_add(y, rms[0], h, rms[1], None, x if x is not h else None)
+        ops.norm_add(y, rms[0], h, rms[1], None, x if x is not h else None, self.residual_scale)
 
     def forward(self, h, step, cache, write_cache=True):
         T, H = h.shape

@@ -39,9 +39,10 @@ class OutputHead(Head):
     graph_safe = True
 
     def __init__(self, vocab_size: int, hidden_size: int, tied_to: TokenEmbedding | None = None, tensor: str = "weight",
-                 scale: float = 1.0):
+                 scale: float = 1.0, softcap: float = 0.0):
         self.vocab_size, self.hidden_size = int(vocab_size), int(hidden_size)
         self.scale = float(scale)       # a multiplier on the logits, applied in 32-bit
+        self.softcap = float(softcap)   # > 0: the (scaled) logits become softcap * tanh(logits / softcap), in 32-bit
         self.tied_to = tied_to
         self.tensor = tensor
         self._weight: torch.Tensor | None = None
@@ -64,17 +65,21 @@ class OutputHead(Head):
         return (rms is not None and step.act_dtype == torch.bfloat16
                 and ops.gemv_norm_supported(h, rms[0], self.weight, n_rows, gated=False, choices=step.choices))
 
-    def forward(self, x: torch.Tensor, out: torch.Tensor, step=None) -> None:
-        ops.gemm(x, self.weight, out, choices=getattr(step, "choices", None))
+    def _finish(self, out: torch.Tensor) -> None:
         if self.scale != 1.0:
             ops.scale_(out, self.scale)
+        if self.softcap > 0:
+            ops.soft_cap_(out, self.softcap)
+
+    def forward(self, x: torch.Tensor, out: torch.Tensor, step=None) -> None:
+        ops.gemm(x, self.weight, out, choices=getattr(step, "choices", None))
+        self._finish(out)
 
     def forward_normed_rows(self, h: torch.Tensor, rows: torch.Tensor, norm, out: torch.Tensor, step=None) -> None:
         """Logits of the chosen rows of the 32-bit stream, the final norm applied inside the product."""
         weight, eps = norm.fused_rms()
         ops.gemv_norm(h, weight, eps, self.weight, out, rows=rows)
-        if self.scale != 1.0:
-            ops.scale_(out, self.scale)
+        self._finish(out)
 
 
 register_part("embedding", "table", Embedding)

@@ -91,4 +91,32 @@ class GatedMLP(FeedForward):
             ops.window.add_row_bias(out, self.b_down)
 
 
+class SquaredReluMLP(FeedForward):
+    """Feed-forward without a gate: down( max(up(x), 0)^2 ), no biases. The activation is part of the up product's
+    epilogue where the matrix kernels take it."""
+    graph_safe = True
+
+    def __init__(self, hidden_size: int, intermediate_size: int, names: dict | None = None):
+        self.hidden_size, self.intermediate_size = int(hidden_size), int(intermediate_size)
+        self.names = {"up": "up_proj.weight", "down": "down_proj.weight"}
+        if names:
+            self.names.update(names)
+        self.w_up: torch.Tensor | None = None
+        self.w_down: torch.Tensor | None = None
+
+    def param_specs(self):
+        H, FF = self.hidden_size, self.intermediate_size
+        return {self.names["up"]: ParamSpec((FF, H)), self.names["down"]: ParamSpec((H, FF))}
+
+    def load_params(self, get: Getter, placement: Placement) -> None:
+        self.w_up = placement.place_matrix(get(self.names["up"]))
+        self.w_down = placement.place_matrix(get(self.names["down"]))
+
+    def forward(self, x, step, out, accumulate):
+        act = step.buffer("mlp.act", (x.shape[0], self.intermediate_size), x.dtype)
+        ops.gemm_squared_relu(x, self.w_up, act, lambda shape, dtype: step.buffer("mlp.up", shape, dtype), choices=step.choices)
+        ops.gemm(act, self.w_down, out, accumulate, fixed_order=step.fixed_order, choices=step.choices)
+
+
 register_part("feed_forward", "gated_mlp", GatedMLP)
+register_part("feed_forward", "squared_relu_mlp", SquaredReluMLP)

@@ -9,10 +9,13 @@
   original: waves shorter than original / high stay, waves longer than original / low slow down by the factor,
   between the two a linear blend in original / wavelength) or, with a factor alone, all slowed down by it;
 * `qk_norm`: every query and key head is divided by its root mean square and multiplied by a weight over the
-  head's entries ("q.norm", "k.norm", shared by all heads) before it is rotated;
+  head's entries ("q.norm", "k.norm", shared by all heads) before it is rotated; `qk_norm="unit"`: divided only, no
+  weight (in front of the rotation or behind it: a rotation leaves a head's length as it is);
 * `softcap` > 0: score <- softcap * tanh(score / softcap);
 * `window` > 0: a query at position p sees keys j with p - j < window, and with `keep_first` also the first
   keep_first tokens of the sequence, at their true positions;
+* `chunk` > 0 (in place of a window): a query at position p sees the keys j <= p with floor(j / chunk) = floor(p / chunk),
+  chunks counted from the sequence's start whatever portions a prompt arrives in;
 * `gate`: the joined heads are multiplied element by element with sigmoid(Wg x) ("g") before the output matrix;
   `gate="heads"`: Wg has one row a head, and a head's whole result is multiplied by its one sigmoid;
 * `sink`: a learned number per head ("sink") whose exponential joins the softmax's denominator: a key that is
@@ -30,7 +33,8 @@
 
 Angles, norms, scores, weights and sums over keys are 32-bit; q and the cached k and v are kept in the activation
 type. What is cached: k [kv_heads * maps, page, dim] after norm and rotation, v [kv_heads, vdim, page]. With a
-window and nothing kept the cache gives pages back as the window passes; kept first tokens make it a full cache.
+window and nothing kept the cache gives pages back as the window passes, with chunks when the next one starts; kept first
+tokens make it a full cache.
 """
 from __future__ import annotations
 
@@ -62,10 +66,10 @@ def banded_frequencies(rot_dims: int, base: float, scaling: dict | None) -> torc
 class WindowAttention(ProjectedMixer):
     def __init__(self, hidden_size: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, rot_dims: int = 0,
                  rot_base: float = 10000.0, rot_scaling: dict | None = None, window: int = 0, keep_first: int = 0,
-                 softcap: float = 0.0, values: str = "projected", gate: bool | str = False, maps: int = 1, qk_norm: bool = False,
+                 softcap: float = 0.0, values: str = "projected", gate: bool | str = False, maps: int = 1, qk_norm: bool | str = False,
                  eps: float = 1e-6, diff: float = 0.0, rot_pairs: str = "halves", sink: bool = False,
                  q_temp: tuple[float, int] | None = None, distance_bias: float = 0.0, own_kv: bool = True,
-                 cache_window: int | None = None):
+                 cache_window: int | None = None, chunk: int = 0):
         if heads % kv_heads:
             raise ValueError(f"{heads} query heads do not divide into {kv_heads} key/value heads")
         if rot_dims % 2 or not 0 <= rot_dims <= dim:
@@ -80,6 +84,10 @@ class WindowAttention(ProjectedMixer):
             raise ValueError("the element-wise gate and two score maps do not go together")
         if window < 0 or keep_first < 0 or (keep_first and not window):
             raise ValueError("keep_first needs a window")
+        if chunk < 0 or (chunk and (window or keep_first or not own_kv or cache_window)):
+            raise ValueError("chunks take the place of a window, in a layer that reads its own keys")
+        if qk_norm not in (False, True, "unit"):
+            raise ValueError(f"qk_norm {qk_norm!r} is none of False, True (with weights) and 'unit' (without)")
         if rot_pairs not in ("halves", "neighbours"):
             raise ValueError(f"rot_pairs {rot_pairs!r} is neither 'halves' nor 'neighbours'")
         if gate not in (False, True, "heads"):
@@ -97,8 +105,9 @@ class WindowAttention(ProjectedMixer):
         self.scale, self.softcap = float(scale), float(softcap)
         self.rot_dims, self.rot_base = int(rot_dims), float(rot_base)
         self.rot_scaling = dict(rot_scaling) if rot_scaling else None
-        self.window, self.keep_first = int(window), int(keep_first)
+        self.window, self.keep_first, self.chunk = int(window), int(keep_first), int(chunk)
         self.values, self.gate, self.maps, self.qk_norm = values, gate, int(maps), bool(qk_norm)
+        self.norm_weights = self.qk_norm and qk_norm != "unit"
         self.rot_pairs, self.sink, self.own_kv = rot_pairs, bool(sink), bool(own_kv)
         self.q_temp = (float(q_temp[0]), int(q_temp[1])) if q_temp is not None else None
         self.distance_bias = float(distance_bias)
@@ -131,7 +140,7 @@ class WindowAttention(ProjectedMixer):
         H = self.hidden_size
         out = {name: ParamSpec((rows, H)) for name, rows in self.input_names()}
         out["o"] = ParamSpec((H, self.out_width))
-        if self.qk_norm:
+        if self.norm_weights:
             out["q.norm"] = ParamSpec((self.dim,), "norm")
             if self.own_kv:
                 out["k.norm"] = ParamSpec((self.dim,), "norm")
@@ -151,7 +160,8 @@ class WindowAttention(ProjectedMixer):
         if not self.own_kv:
             return None
         slides = self.cache_window > 0 and self.keep_first == 0
-        return CacheSpec(kind="window" if slides else "full", window=self.cache_window if slides else 0,
+        kind, length = ("chunk", self.chunk) if self.chunk else ("window", self.cache_window) if slides else ("full", 0)
+        return CacheSpec(kind=kind, window=length,
                          paged={"k": (self.kv_heads * self.maps, PAGE, self.dim), "v": (self.kv_heads, self.vdim, PAGE)})
 
     def load_core(self, get: Getter, placement: Placement) -> None:
@@ -159,7 +169,7 @@ class WindowAttention(ProjectedMixer):
         if self.rot_dims:
             # frequencies in 64-bit, stored in 32-bit; the angle is the kernel's 32-bit product with the position
             self.inv_freq = placement.place(banded_frequencies(self.rot_dims, self.rot_base, self.rot_scaling).to(f32), f32)
-        if self.qk_norm:
+        if self.norm_weights:
             self.wq = placement.place(get("q.norm"), f32)
             self.wk = placement.place(get("k.norm"), f32) if self.own_kv else None
         if self.sink:
@@ -185,12 +195,13 @@ class WindowAttention(ProjectedMixer):
         table = step.block_tables[cache.group]
         k_cache, v_cache = cache.paged["k"], cache.paged["v"]
         q = step.buffer("window_attention.q", (T, nq * dim), step.act_dtype)
+        unit = self.qk_norm and not self.norm_weights
         if own:
             ops.window.qk_prepare(p, step, table, q, k_cache, v_cache, nq, k_col, v_col, self.inv_freq, self.rot_dims,
-                                  self.wq, self.wk, self.eps, self.rot_pairs, self.q_temp)
+                                  self.wq, self.wk, self.eps, self.rot_pairs, self.q_temp, unit_norm=unit)
         else:
             ops.window.qk_prepare(p, step, None, q, None, None, nq, 0, None, self.inv_freq, self.rot_dims, self.wq, None,
-                                  self.eps, self.rot_pairs, self.q_temp, dk=dim)
+                                  self.eps, self.rot_pairs, self.q_temp, dk=dim, unit_norm=unit)
         # what is done with the runs' parts; where the keys are in one run the attention kernel may do it itself
         if M == 2:
             finish = dict(out=o, mode="difference", lam=self.lam, eps=self.eps, out_scale=(1.0 - self.diff) * scale)
@@ -201,7 +212,7 @@ class WindowAttention(ProjectedMixer):
         else:
             finish = dict(out=o, mode="plain", out_scale=scale, sinks=self.sinks)
         parts = ops.window.window_attention(q, k_cache, v_cache, step, table, nq, self.scale, self.softcap, self.window,
-                                            self.keep_first, self.slopes, finish=finish)
+                                            self.keep_first, self.slopes, finish=finish, chunk=self.chunk)
         if parts != "finished":
             out = finish.pop("out")
             ops.window.window_attention_finish(parts[0], parts[1], out, n, **finish)

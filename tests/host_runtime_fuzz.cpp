@@ -12,7 +12,7 @@
 #include <vector>
 
 extern "C" {
-void* llme_cm_create(int n_groups, const int* is_window, const int* window, const int* num_pages, int page_size,
+void* llme_cm_create(int n_groups, const int* kind, const int* window, const int* num_pages, int page_size,
                      int max_requests);
 void llme_cm_destroy(void* h);
 int llme_cm_admit(void* h, int64_t key);
@@ -70,9 +70,9 @@ static int pick(int lo, int hi) { return std::uniform_int_distribution<int>(lo, 
 static void fuzz_cache_manager(int rounds) {
     for (int round = 0; round < rounds; ++round) {
         const int page = 1 << pick(0, 5), slots = pick(1, 9), window = pick(1, 70);
-        const int is_window[2] = {0, 1}, win[2] = {0, window}, pages[2] = {pick(4, 60), pick(4, 60)};
+        const int kind[2] = {0, pick(1, 2)}, win[2] = {0, window}, pages[2] = {pick(4, 60), pick(4, 60)};
         const int G = pick(1, 2);
-        void* cm = llme_cm_create(G, is_window, win, pages, page, slots);
+        void* cm = llme_cm_create(G, kind, win, pages, page, slots);
         REQUIRE(cm != nullptr);
         std::map<int64_t, long> length;                       // what this driver believes
         std::vector<int> done;
@@ -171,8 +171,8 @@ static void fuzz_cache_manager(int rounds) {
 static void fuzz_scheduler(int rounds) {
     for (int round = 0; round < rounds; ++round) {
         const int page = 1 << pick(1, 4), max_concurrent = pick(1, 6), budget = pick(1, 40);
-        const int is_window[1] = {0}, win[1] = {0}, pages[1] = {pick(3, 40)};
-        void* cm = llme_cm_create(1, is_window, win, pages, page, max_concurrent);
+        const int kind[1] = {0}, win[1] = {0}, pages[1] = {pick(3, 40)};
+        void* cm = llme_cm_create(1, kind, win, pages, page, max_concurrent);
         void* sc = llme_sched_create(cm, max_concurrent, budget);
         REQUIRE(cm && sc);
         REQUIRE(llme_sched_set_decode_round(sc, -1) < 0 && llme_sched_set_decode_round(sc, pick(0, 4)) == 0);

@@ -12,7 +12,8 @@ step never fails for capacity half-way.
 
 Layers with the same needs form a group with a page pool and block tables of its
 own: a "full" group keeps every token of a request; a "window" group gives pages
-back once every position in them lies behind the window of the next token. Beside
+back once every position in them lies behind the window of the next token; a "chunk" group
+once the next token's own stretch of `window` positions (counted from 0) starts behind them. Beside
 the pages, every live request holds a slot: a row in each fixed-size state tensor.
 """
 from __future__ import annotations
@@ -60,7 +61,7 @@ class PagePool:
 @dataclass(frozen=True)
 class GroupSpec:
     name: str
-    kind: str = "full"          # "full" | "window"
+    kind: str = "full"          # "full" | "window" | "chunk"
     window: int = 0
     num_pages: int = 0
 
@@ -83,10 +84,10 @@ class CacheManager:
         if len(set(names)) != len(names):
             raise ValueError(f"cache groups must have distinct names, got {names}")
         for g in groups:
-            if g.kind not in ("full", "window"):
-                raise ValueError(f"group {g.name}: kind {g.kind!r} is not 'full' or 'window'")
-            if g.kind == "window" and g.window <= 0:
-                raise ValueError(f"group {g.name}: a window group needs window > 0")
+            if g.kind not in ("full", "window", "chunk"):
+                raise ValueError(f"group {g.name}: kind {g.kind!r} is not 'full', 'window' or 'chunk'")
+            if g.kind != "full" and g.window <= 0:
+                raise ValueError(f"group {g.name}: a {g.kind} group needs window > 0")
         self.page_size = int(page_size)
         self.max_requests = int(max_requests)
         self.groups = {g.name: g for g in groups}
@@ -130,6 +131,8 @@ class CacheManager:
         """First logical block that a token at `position` reads in this group."""
         if group.kind == "window":
             return max(0, position - group.window + 1) // self.page_size
+        if group.kind == "chunk":
+            return (position - position % group.window) // self.page_size
         return 0
 
     def _missing(self, req: _Request, group: GroupSpec, n_new: int) -> list[int]:
@@ -217,7 +220,7 @@ class CacheManager:
             raise CacheError(f"request {request_id!r}: commit of {n_new} tokens beyond the reserved pages")
         req.length += n_new
         for g in self.groups.values():
-            if g.kind != "window":
+            if g.kind == "full":
                 continue
             table = req.tables[g.name]
             keep_from = self._first_needed_block(g, req.length)     # next token's first block

@@ -79,6 +79,31 @@ def test_window_group_gives_pages_back():
     assert m.free_pages("win") == 64 and m.free_pages("full") == 64
 
 
+def test_chunk_group_gives_pages_back_when_the_next_token_starts_a_chunk():
+    m = CacheManager([GroupSpec("full", "full", 0, 64), GroupSpec("c", "chunk", 10, 64)], page_size=4, max_requests=1)
+    m.admit("r")
+    assert m.reserve("r", 9)
+    m.commit("r", 9)                       # the next token, 9, still belongs to positions 0..9
+    assert [p >= 0 for p in m.block_table("r", "c")] == [True] * 3
+    assert m.reserve("r", 1)
+    m.commit("r", 1)                       # the next token, 10, starts a chunk; block 2 holds 8..11 and stays
+    assert [p >= 0 for p in m.block_table("r", "c")] == [False, False, True]
+    assert m.reserve("r", 25)              # a portion over several chunks gets pages for all its own tokens
+    m.commit("r", 25)                      # 35 tokens: the next token's chunk is 30..39, blocks 7 (28..31) and 8
+    assert [b for b, p in enumerate(m.block_table("r", "c")) if p >= 0] == [7, 8]
+    assert m.free_pages("c") == 62
+    for n in range(36, 90):
+        assert m.reserve("r", 1)
+        m.commit("r", 1)
+        m.check()
+        first = n // 10 * 10 // 4
+        assert [b for b, p in enumerate(m.block_table("r", "c")) if p >= 0] == list(range(first, (n - 1) // 4 + 1))
+    m.release("r")
+    assert m.free_pages("c") == 64
+    with pytest.raises(ValueError, match="chunk"):
+        CacheManager([GroupSpec("c", "chunk", 0, 4)], page_size=4, max_requests=1)
+
+
 def test_slots():
     m = CacheManager([GroupSpec("full", "full", 0, 4)], page_size=4, max_requests=2)
     s0, s1 = m.admit("a"), m.admit("b")
@@ -100,7 +125,7 @@ def test_random_orders_keep_the_invariants(seed):
     rng = random.Random(seed)
     groups = [GroupSpec("full", "full", 0, 40)]
     if seed % 2:
-        groups.append(GroupSpec("win", "window", rng.choice([3, 8, 17]), 25))
+        groups.append(GroupSpec("win", "window" if seed % 4 == 1 else "chunk", rng.choice([3, 8, 17]), 25))
     m = CacheManager(groups, page_size=rng.choice([1, 4, 16]), max_requests=5)
     live: dict[int, int] = {}
     next_id = 0
@@ -131,7 +156,8 @@ def test_random_orders_keep_the_invariants(seed):
         for rid, n in live.items():                               # every readable key has a page
             for g in m.groups.values():
                 table = m.block_table(rid, g.name)
-                lo = max(0, n - g.window + 1) if g.kind == "window" else 0   # the next token at n reads keys > n - window
+                # the next token at n reads keys > n - window, or those of its own chunk
+                lo = max(0, n - g.window + 1) if g.kind == "window" else n // g.window * g.window if g.kind == "chunk" else 0
                 for pos in range(lo, n):
                     assert table[pos // m.page_size] >= 0
     for rid in list(live):
@@ -183,6 +209,8 @@ def test_native_manager_agrees_with_the_plain_one(seed):
     specs = [("full", "full", 0, rng.choice([9, 30])), ("win", "window", rng.choice([2, 7, 20]), rng.choice([6, 18]))]
     if seed % 3 == 0:
         specs = specs[:1]
+    if seed % 3 == 1:
+        specs.append(("chunk", "chunk", rng.choice([3, 8, 21]), rng.choice([7, 20])))
     page = rng.choice([1, 4, 16])
     a = CacheManager([GroupSpec(*s) for s in specs], page, 4)
     b = plain_cache.CacheManager([plain_cache.GroupSpec(*s) for s in specs], page, 4)
