@@ -23,7 +23,9 @@ a residual in several streams) beside Llama with layers of the same sizes: prefi
 with biases and clamped experts chosen by a table, a stretch of layers that runs two passes),
 `--design zapolorn` the Zapolorn design (sublayers normed behind; windowed attention with sinks and head gates, one layer in
 three reading the keys of the layer in front; attention with a bias by distance beside a gated linear attention; dense
-feed-forwards and experts that weigh their input).
+feed-forwards and experts that weigh their input),
+`--design lukupel` the Lukupel design (sublayers normed behind; a matrix memory with exponential gates, and attention within
+chunks of the sequence; feed-forwards with a squared rectifier).
 
 `--phase mixed` times one step of continuous batching (a prompt portion beside decoded tokens of
 other requests), `--phase portion` portions of one long prompt. `--phase serve` is another workload (with `--shape 3b`: 32 requests with prompts of 64 to 3,072
@@ -171,6 +173,24 @@ def zapolorn_at(width: int, ff: int, heads: int, layers: int, vocab: int, only: 
             "logit_scale": 1.0, "layers": out}
 
 
+def lukupel_at(width: int, ff: int, heads: int, layers: int, vocab: int, only: str = "") -> dict:
+    """Lukupel layers of a Llama layer's width and bytes of weights: the matrix memory (a quarter as many heads, keys of 128
+    over values of 256, so that the values have the layer's width), then two of attention within chunks of 1,024 (heads of 64,
+    a quarter as many key heads, half of a head rotated), every one with a feed-forward of two matrices of one and a half
+    times the size, which are as many weights as Llama's three."""
+    dense = {"kind": "dense", "ff": ff * 3 // 2}
+    memory = {"heads": max(1, heads // 4), "dim": 128, "vdim": 256, "gate_cap": 12.0}
+    chunked = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 64, "vdim": 64, "scale": 0.3, "mask": {"size": 1024},
+               "rot": {"base": 500000.0, "dims": 32, "scaling": {"factor": 8.0}}}
+    kinds = {"mlstm": {"type": "mlstm", "mixer": memory, "mlp": dense}, "chunked": {"type": "attention", "mixer": chunked, "mlp": dense}}
+    return {"architecture": "Lukupel", "vocab": vocab, "width": width, "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6},
+            "residual_mult": 1.0, "logit_softcap": 30.0,
+            "layers": [kinds[only or ("mlstm", "chunked", "chunked")[i % 3]] for i in range(layers)]}
+
+
+DESIGNS = {"rilonex": rilonex_at, "bidirax": bidirax_at, "zetonex": zetonex_at, "zapolorn": zapolorn_at, "lukupel": lukupel_at}
+
+
 def design(args) -> int:
     """Prefill (one prompt of --prefill-tokens) and decode (--batch requests at --context) of the Rilonex design and of
     Llama with layers of the same width, feed-forward size and number of heads: tokens/s of both and their ratio, per
@@ -183,10 +203,7 @@ def design(args) -> int:
     for size in [x for x in args.design_sizes.split(",") if x]:
         width, ff, heads = DESIGN_SIZES[size]
         row = {"size": size, "width": width, "ff": ff, "heads": heads, "layers": layers}
-        other = (bidirax_at(width, ff, heads, layers, vocab, only=args.design_only) if args.design == "bidirax"
-                 else zetonex_at(width, ff, heads, layers, vocab, only=args.design_only) if args.design == "zetonex"
-                 else zapolorn_at(width, ff, heads, layers, vocab, only=args.design_only) if args.design == "zapolorn"
-                 else rilonex_at(width, ff, heads, layers, vocab, only=args.design_only))
+        other = DESIGNS[args.design](width, ff, heads, layers, vocab, only=args.design_only)
         for name, cfg in (("llama", llama_at(width, ff, heads, layers, vocab)), (args.design, other)):
             if args.design_skip_llama and name == "llama":
                 continue
@@ -429,11 +446,12 @@ def main() -> int:
                          "steps of --portion prompt tokens of one request behind --context tokens; 'mixed': such a "
                          "portion beside one decoded token of --batch other requests")
     ap.add_argument("--design-sizes", default="1k,2k", help="design: sizes to run, of " + ",".join(sorted(DESIGN_SIZES)))
-    ap.add_argument("--design", default="rilonex", choices=["rilonex", "bidirax", "zetonex", "zapolorn"],
+    ap.add_argument("--design", default="rilonex", choices=sorted(DESIGNS),
                     help="design: which design runs beside Llama")
-    ap.add_argument("--design-only", default="", choices=["", "rglru", "channel_delta", "parallel", "rotated", "windowed", "differential", "gated"],
-                    help="design: a model of this kind of layer only (the first three Rilonex, the next two Bidirax, the last "
-                         "two Zetonex; Zapolorn: windowed or parallel)")
+    ap.add_argument("--design-only", default="", choices=["", "rglru", "channel_delta", "parallel", "rotated", "windowed", "differential", "gated", "mlstm",
+                                                             "chunked"],
+                    help="design: a model of this kind of layer only (the first three Rilonex, the next two Bidirax, two "
+                         "more Zetonex, the last two Lukupel; Zapolorn: windowed or parallel)")
     ap.add_argument("--design-skip-llama", action="store_true", help="design: time the design alone")
     ap.add_argument("--portion", type=int, default=256, help="portion: prompt tokens a step")
     ap.add_argument("--decode-len", type=int, default=700, help="mixed: tokens of the shortest decoding request "

@@ -10,11 +10,28 @@ norms standing behind them. A layer may borrow all tensors of another one; what 
 """
 from __future__ import annotations
 
+import contextlib
 import math
 
 import torch
 
 F64 = torch.float64
+
+
+# What a model of narrower storage keeps between its kernels (inputs of matrix products, the attention's and the memory's
+# queries, keys and values) passes through here; the identity unless `bfloat16_storage` is in force.
+_kept = lambda x: x
+
+
+@contextlib.contextmanager
+def bfloat16_storage():
+    """Inside, those values are rounded to bfloat16: what rounding alone makes of a model's logits."""
+    global _kept
+    _kept = lambda x: x.to(torch.bfloat16).to(F64)
+    try:
+        yield
+    finally:
+        _kept = lambda x: x
 
 
 def rms_unit(x: torch.Tensor, eps: float) -> torch.Tensor:
@@ -27,7 +44,7 @@ def norm(x, w, eps):
 
 
 def linear(x, w, b=None):
-    y = x @ w.to(F64).T
+    y = _kept(x) @ w.to(F64).T
     return y if b is None else y + b.to(F64)
 
 
@@ -68,6 +85,7 @@ def attend(q, k, v, scale, mask):
     """q [T, n, d], k [T, g, d], v [T, g, dv] -> [T, n, dv]; head h reads key/value head h // (n // g)."""
     T, n, _ = q.shape
     g = k.shape[1]
+    q, k, v = _kept(q), _kept(k), _kept(v)
     out = torch.zeros(T, n, v.shape[2], dtype=F64)
     for h in range(n):
         kv = h // (n // g)
@@ -110,6 +128,7 @@ def matrix_memory(q, k, v, i, f, state=None):
     o = S'^T q / (max(|z' . q|, e^(-m')) + 1e-6). Returns (o [T, n, dv], (S, z, m))."""
     T, n, d = q.shape
     dv = v.shape[2]
+    q, k, v = _kept(q), _kept(k), _kept(v)
     if state is None:
         state = (torch.zeros(n, d, dv, dtype=F64), torch.zeros(n, d, dtype=F64), torch.zeros(n, dtype=F64))
     S, z, m = state
