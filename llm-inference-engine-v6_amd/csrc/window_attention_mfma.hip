@@ -111,6 +111,8 @@ __device__ __forceinline__ float capped_score(float s, float k, float cap) {
 template <int NVM, bool EDGE, int CAP>
 __device__ __forceinline__ void window_block(const WindowArgs& a, const f32x4 (&sc)[2], bf16x8 (&vf)[NVM], f32x4 (&acc)[NVM], float& m,
                                              float& l, int nvt, int key0, int qd, int pos, int lo, int pos_max, bool valid, float inv_cap, float slope) {
+    // (the kernel without LDS and the staged one give the same bits: no product is merged into a sum in one and not in the other)
+#pragma clang fp contract(off)
     float p[8];
     float mx = -INFINITY;
 #pragma unroll
@@ -298,6 +300,7 @@ __global__ __launch_bounds__(256, (DSM <= 2 && NVM <= 4) ? 4 : NVM <= 4 ? 3 : 2)
 template <int NVM, bool EDGE, int CAP>
 __device__ __forceinline__ void shared_block(const WindowArgs& a, const f32x4 (&sc)[2], const bf16* lds_v, f32x4 (&acc)[NVM], float& m,
                                              float& l, int nvt, int key0, int r, int qd, int pos, int lo, bool valid, float inv_cap, float slope) {
+#pragma clang fp contract(off)
     float p[8];
     float mx = -INFINITY;
 #pragma unroll

@@ -174,10 +174,12 @@ def test_the_matrix_core_attention_at_other_sizes(tmp_path, name):
 
 
 @pytest.mark.parametrize("name", sorted(MATRIX_CORES))
-def test_staged_blocks_of_keys_give_what_a_wavefront_alone_gives(tmp_path, name):
+def test_staged_blocks_of_keys_give_what_a_wavefront_alone_gives(tmp_path, name, monkeypatch):
     """Prompts' attention with every block of keys staged once a workgroup through LDS walks the same blocks in the same
-    order as the kernel in which a wavefront fetches its own: the logits agree to the last bits, whole and in portions."""
+    order as the kernel in which a wavefront fetches its own: the logits agree to the last bits, whole and in portions.
+    (Keys in one run: cut into several, one kernel cuts a workgroup's blocks and the other a tile's, at other places.)"""
     from llmengine.ops import window
+    monkeypatch.setattr(window, "WINDOW_MFMA_MAX_RUNS", 1)
     cfg = MATRIX_CORES[name]
     engine, weights = _engine(tmp_path, cfg, 22, "bf16")
     V = cfg["vocab"]
