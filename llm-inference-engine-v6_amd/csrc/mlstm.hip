@@ -10,7 +10,8 @@
 // that is always 1), and level [heads, vdim + 1], a copy of m for every column, so that whoever walks a column needs
 // nothing that another workgroup writes.
 //
-// Two ways through a request's rows, chosen by how many it brings to the step (`chunk_from`: that many or more are chunked).
+// A step in which every request brings one row has a kernel of its own (memory, division, norm and gate in one workgroup a
+// head). Otherwise two ways through a request's rows, chosen by how many it brings (`chunk_from`: that many or more are chunked).
 // The walk (any sizes, 32-bit throughout; decoded tokens, short portions, the 32-bit model) takes them one by one, columns
 // side by side. The chunked form (bfloat16 model, long portions) uses that the rule is linear in S: with b_t the sum of f up to row t of a chunk, a_t = i_t - b_t and M_t = max(m_start, a_1 .. a_t),
 //   m_t = b_t + M_t,   S_t = e^(m_start - M_t) S_start + sum_(s <= t) e^(a_s - M_t) k_s v_s^T,
@@ -192,6 +193,91 @@ __global__ __launch_bounds__(256) void mlstm_finish_kernel(const float* __restri
     for (int j = lane; j < vdim; j += kWave) {
         const float z = g[static_cast<size_t>(t) * ld_g + h * vdim + j];
         out[static_cast<size_t>(t) * ld_out + h * vdim + j] = from_float<TO>((p[j] * inv) * w[h * vdim + j] / (1.0f + expf(-z)));
+    }
+}
+
+// A step in which every request brings one row (decoding): one workgroup of 1,024 threads per (request, head) takes the row
+// through the whole memory and finishes it, so that nothing is passed on. 16 lanes share a column (R key channels each), 64
+// columns a pass, four passes' columns asked for together. VEC: channels come in whole pieces of four.
+template <int R, bool VEC, typename TO>
+__global__ __launch_bounds__(1024) void mlstm_single_kernel(MlstmInput in, float* __restrict__ memory, float* __restrict__ level,
+                                                            const int* __restrict__ slots, const float* __restrict__ norm_w, int g_col,
+                                                            float eps, float scale, TO* __restrict__ out, int ld_out) {
+    constexpr int COLS = 64, U = R >= 16 ? 2 : 4;
+    extern __shared__ float read_s[];                       // [vdim + 1]
+    __shared__ float scratch[16];
+    const int t = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
+    const int cl = tid >> 4, l = tid & 15, vdim = in.vdim, dim = in.dim;
+    const float* row = in.p + static_cast<size_t>(t) * in.ld;
+    const size_t column0 = (static_cast<size_t>(slots[t]) * in.heads + h) * (vdim + 1);
+    float kk[R], qq[R];
+    auto load = [&](const float* src, float (&dst)[R]) {
+        if constexpr (VEC) {
+#pragma unroll
+            for (int i = 0; i < R; i += 4) {
+                float4 x{0.f, 0.f, 0.f, 0.f};
+                if (l * R + i < dim) x = *reinterpret_cast<const float4*>(src + l * R + i);
+                dst[i] = x.x; dst[i + 1] = x.y; dst[i + 2] = x.z; dst[i + 3] = x.w;
+            }
+        } else {
+#pragma unroll
+            for (int i = 0; i < R; ++i) dst[i] = l * R + i < dim ? src[l * R + i] : 0.f;
+        }
+    };
+    load(row + in.k_col + h * dim, kk);
+    load(row + in.q_col + h * dim, qq);
+    const float li = capped_gate(row[in.i_col + h] + in.bias[h], in.cap);
+    const float lf = log_sigmoid(capped_gate(row[in.f_col + h] + in.bias[in.heads + h], in.cap));
+    const float lev = level[column0];                       // (a copy for every column; this workgroup is the only one that takes them)
+    const float top = fmaxf(lf + lev, li);
+    const float keep = expf(lf + lev - top), add = expf(li - top);
+    for (int c0 = 0; c0 < vdim; c0 += COLS * U) {
+        // (place U of the first pass: the key sum, column vdim, by the first sixteen lanes)
+        float m[U + 1][R], vv[U + 1];
+#pragma unroll
+        for (int u = 0; u <= U; ++u) {
+            const int c = u < U ? c0 + u * COLS + cl : vdim;
+            const bool mine = u < U ? c < vdim : c0 == 0 && cl == 0;
+            vv[u] = mine && u < U ? row[in.v_col + h * vdim + c] : 1.f;
+            if (mine) load(memory + (column0 + c) * dim, m[u]);
+        }
+#pragma unroll
+        for (int u = 0; u <= U; ++u) {
+            const int c = u < U ? c0 + u * COLS + cl : vdim;
+            if (!(u < U ? c < vdim : c0 == 0 && cl == 0)) continue;         // (sixteen neighbouring lanes together)
+            const float w = add * vv[u];
+            float reads[2] = {0.f, 0.f};
+#pragma unroll
+            for (int i = 0; i < R; ++i) {
+                m[u][i] = fmaf(kk[i], w, keep * m[u][i]);
+                reads[i & 1] = fmaf(m[u][i], qq[i], reads[i & 1]);
+            }
+            float* M = memory + (column0 + c) * dim + l * R;
+            if constexpr (VEC) {
+#pragma unroll
+                for (int i = 0; i < R; i += 4)
+                    if (l * R + i < dim) *reinterpret_cast<float4*>(M + i) = float4{m[u][i], m[u][i + 1], m[u][i + 2], m[u][i + 3]};
+            } else {
+#pragma unroll
+                for (int i = 0; i < R; ++i)
+                    if (l * R + i < dim) M[i] = m[u][i];
+            }
+            const float read = sum_of_group<16>(reads[0] + reads[1]) * in.q_scale;
+            if (l == 0) read_s[c] = read;
+        }
+    }
+    __syncthreads();                                        // (every thread has read the level by now)
+    for (int c = tid; c <= vdim; c += 1024) level[column0 + c] = top;
+    const float inv_den = 1.0f / (fmaxf(fabsf(read_s[vdim]), expf(-top)) + 1e-6f);
+    float ss = 0.f;
+    for (int c = tid; c < vdim; c += 1024) {
+        const float v = read_s[c] * inv_den;
+        ss = fmaf(v, v, ss);
+    }
+    const float inv = scale * inv_den / sqrtf(block_sum(ss, scratch, 16) / static_cast<float>(vdim) + eps);
+    for (int c = tid; c < vdim; c += 1024) {
+        const float z = row[g_col + h * vdim + c];
+        out[static_cast<size_t>(t) * ld_out + h * vdim + c] = from_float<TO>((read_s[c] * inv) * norm_w[h * vdim + c] / (1.0f + expf(-z)));
     }
 }
 
@@ -415,9 +501,9 @@ __global__ __launch_bounds__(256) void mlstm_chunk_carry_kernel(float* __restric
     const size_t column = (static_cast<size_t>(slots[s]) * heads + h) * (vdim + 1) + col;
     float4* slot = reinterpret_cast<float4*>(memory + column * dim + d);
     float4 S = *slot;
-    float m = level[column];            // (the new one is the next kernel's: other threads of the column still read this one)
+    float m = level[column];            // (the next kernel writes the new one: other threads still read this one)
     size_t at = static_cast<size_t>(chunk_place(q_start, s, 0)) * heads + h;
-    constexpr int AHEAD = 4;
+    constexpr int AHEAD = 8;
     for (int c0 = 0; c0 < nc; c0 += AHEAD) {
         float4 add[AHEAD];
         float end[AHEAD], top[AHEAD];
@@ -459,26 +545,15 @@ __global__ __launch_bounds__(256) void mlstm_chunk_carry_kernel(float* __restric
     *slot = S;
 }
 
-// level of every column behind the step's rows, from the chunks' ends (the same recurrence as above).
-__global__ __launch_bounds__(256) void mlstm_chunk_level_kernel(float* __restrict__ level, const int* __restrict__ q_start,
-                                                                const int* __restrict__ slots, int heads, int vdim, MlstmChunks ck) {
-    const int s = blockIdx.y, h = blockIdx.x;
-    const int rows = q_start[s + 1] - q_start[s];
-    const int nc = (rows + kChunk - 1) / kChunk;
-    if (nc <= 0 || rows < ck.chunk_from) return;
-    const size_t z = (static_cast<size_t>(chunk_place(q_start, s, 0)) + nc - 1) * heads + h;
-    const float m = ck.ends[z * 2] + fmaxf(ck.m[z], ck.ends[z * 2 + 1]);
-    float* lev = level + (static_cast<size_t>(slots[s]) * heads + h) * (vdim + 1);
-    for (int c = threadIdx.x; c <= vdim; c += 256) lev[c] = m;
-}
-
 // The rows of half a chunk (64) of one head: NW wavefronts, wavefront w the value tiles w, w + NW, .. (NCT of them) over
 // all 64 rows, so that the memory and the values are each read once. Products as in the attention kernels: the first
 // operand's rows are what is made (values, keys), the second operand's columns are the rows t; a lane ends up with row
-// t = 16 rt + r. LDS: Q and K [64][DP + 8], V^T [16 tiles][64 + 8], the weights in two parts [64][64 + 8].
-template <int NW, int NCT>
+// t = 16 rt + r. LDS: Q and K [64][DP + 8], V^T [16 tiles][64 + 8], the weights in two parts [64][64 + 8]. DS: slabs of 32
+// key channels. Everything the first products need is asked for before anything waits; the workgroup of a request's last
+// chunk also leaves the slot's new level.
+template <int NW, int NCT, int DS>
 __global__ __launch_bounds__(NW * 64) void mlstm_chunk_read_kernel(MlstmInput in, const int* __restrict__ q_start, int n_chunks,
-                                                                   MlstmChunks ck, const float* __restrict__ norm_w, int g_col, float eps,
+                                                                   const int* __restrict__ slots, float* __restrict__ level, MlstmChunks ck, const float* __restrict__ norm_w, int g_col, float eps,
                                                                    float scale, bf16* __restrict__ out, int ld_out) {
     constexpr int NT = NW * 64, KB = 64, KS = KB + 8;
     extern __shared__ __align__(16) unsigned char lds_raw[];
@@ -494,52 +569,99 @@ __global__ __launch_bounds__(NW * 64) void mlstm_chunk_read_kernel(MlstmInput in
     const size_t z = static_cast<size_t>(chunk_place(q_start, s, c)) * in.heads + h;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, qd = lane >> 4;
     const int dim = in.dim, vdim = in.vdim;
-    const int ds = (dim + 31) >> 5, DP = ds * 32, QS = DP + 8, nvt = vdim >> 4;
+    constexpr int DP = DS * 32, QS = DP + 8;
+    const int nvt = vdim >> 4;
     bf16* q_l = reinterpret_cast<bf16*>(lds_raw);
     bf16* k_l = q_l + 64 * QS;
     bf16* v_l = k_l + KB * QS;
     bf16* p_hi = v_l + vdim * KS;
     bf16* p_lo = p_hi + 64 * KS;
 
-    // rows [first, first + 64) of the chunk's q or k into LDS, behind `count` and behind `dim` zeros
-    auto stage_rows = [&](bf16* dst, int col, int first, int count) {
-        const int per = DP / 4;
-        for (int item = tid; item < 64 * per; item += NT) {
-            const int row = item / per, d = (item % per) * 4;
-            float4 x{0.f, 0.f, 0.f, 0.f};
-            if (row < count && d < dim)
-                x = *reinterpret_cast<const float4*>(in.p + static_cast<size_t>(t_chunk + first + row) * in.ld + col + h * dim + d);
+    // rows [first, first + 64) of the chunk's q or k: pieces of four entries, zeros behind `count` and behind `dim`
+    constexpr int PER = DP / 4, QI = 64 * PER / NT;
+    auto load_rows = [&](float4 (&x)[QI], int col, int first, int count) {
+#pragma unroll
+        for (int i = 0; i < QI; ++i) {
+            const int item = tid + NT * i, row = item / PER, d = (item % PER) * 4;
+            x[i] = (row < count && d < dim)
+                       ? *reinterpret_cast<const float4*>(in.p + static_cast<size_t>(t_chunk + first + row) * in.ld + col + h * dim + d)
+                       : float4{0.f, 0.f, 0.f, 0.f};
+        }
+    };
+    auto put_rows = [&](bf16* dst, const float4 (&x)[QI]) {
+#pragma unroll
+        for (int i = 0; i < QI; ++i) {
+            const int item = tid + NT * i, row = item / PER, d = (item % PER) * 4;
             bf16x4 y;
-            y[0] = static_cast<bf16>(x.x);
-            y[1] = static_cast<bf16>(x.y);
-            y[2] = static_cast<bf16>(x.z);
-            y[3] = static_cast<bf16>(x.w);
+            y[0] = static_cast<bf16>(x[i].x);
+            y[1] = static_cast<bf16>(x[i].y);
+            y[2] = static_cast<bf16>(x[i].z);
+            y[3] = static_cast<bf16>(x[i].w);
             *reinterpret_cast<bf16x4*>(dst + row * QS + d) = y;
         }
     };
-    // values of rows [first, first + 64), turned round
-    auto stage_values = [&](int first, int count) {
-        for (int item = tid; item < 16 * (vdim / 4); item += NT) {
-            const int sg = item & 15, e0 = (item >> 4) * 4;
+    // values of rows [first, first + 64), pieces of four rows by four entries, turned round as they are stored
+    constexpr int VI = NCT;
+    auto load_values = [&](float4 (&x)[VI][4], int first, int count) {
+#pragma unroll
+        for (int i = 0; i < VI; ++i) {
+            const int item = tid + NT * i, sg = item & 15, e0 = (item >> 4) * 4;
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+                x[i][j] = (e0 < vdim && sg * 4 + j < count)
+                              ? *reinterpret_cast<const float4*>(in.p + static_cast<size_t>(t_chunk + first + sg * 4 + j) * in.ld + in.v_col + h * vdim + e0)
+                              : float4{0.f, 0.f, 0.f, 0.f};
+        }
+    };
+    auto put_values = [&](const float4 (&v)[VI][4]) {
+#pragma unroll
+        for (int i = 0; i < VI; ++i) {
+            const int item = tid + NT * i, sg = item & 15, e0 = (item >> 4) * 4;
+            if (e0 >= vdim) continue;
             bf16x4 x[4];
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
-                float4 v{0.f, 0.f, 0.f, 0.f};
-                if (sg * 4 + j < count)
-                    v = *reinterpret_cast<const float4*>(in.p + static_cast<size_t>(t_chunk + first + sg * 4 + j) * in.ld + in.v_col + h * vdim + e0);
-                x[0][j] = static_cast<bf16>(v.x);
-                x[1][j] = static_cast<bf16>(v.y);
-                x[2][j] = static_cast<bf16>(v.z);
-                x[3][j] = static_cast<bf16>(v.w);
+                x[0][j] = static_cast<bf16>(v[i][j].x);
+                x[1][j] = static_cast<bf16>(v[i][j].y);
+                x[2][j] = static_cast<bf16>(v[i][j].z);
+                x[3][j] = static_cast<bf16>(v[i][j].w);
             }
 #pragma unroll
             for (int e = 0; e < 4; ++e) *reinterpret_cast<bf16x4*>(v_l + (e0 + e) * KS + sg * 4) = x[e];
         }
     };
-    stage_rows(q_l, in.q_col, row0, n);
-    for (int d = tid; d < dim; d += NT) z_s[d] = ck.z[z * dim + d];
+    bf16x8 s_hi[NCT][DS], s_lo[NCT][DS];                    // the memory in front of the chunk, this wavefront's columns
     const float m_start = ck.m[z];
-    chunk_gates(in, h, t_chunk, n_chunk, b_s, a_s, M_s, scratch);           // (its barriers also cover q_l and z_s)
+    {
+        float4 xq[QI], xk[QI], xv[VI][4];
+        load_rows(xq, in.q_col, row0, n);
+        load_rows(xk, in.k_col, 0, min(KB, n_chunk));
+        load_values(xv, 0, min(KB, n_chunk));
+#pragma unroll
+        for (int j = 0; j < NCT; ++j) {
+            const int ct = wave + NW * j;
+#pragma unroll
+            for (int k = 0; k < DS; ++k) {
+                const int d0 = k * 32 + qd * 8;
+#pragma unroll
+                for (int e = 0; e < 8; ++e) s_hi[j][k][e] = s_lo[j][k][e] = static_cast<bf16>(0.f);
+                if (ct < nvt && d0 < dim) {
+                    s_hi[j][k] = *reinterpret_cast<const bf16x8*>(ck.s_hi + (z * vdim + ct * 16 + r) * dim + d0);
+                    s_lo[j][k] = *reinterpret_cast<const bf16x8*>(ck.s_lo + (z * vdim + ct * 16 + r) * dim + d0);
+                }
+            }
+        }
+        put_rows(q_l, xq);
+        put_rows(k_l, xk);
+        put_values(xv);
+    }
+    for (int d = tid; d < dim; d += NT) z_s[d] = ck.z[z * dim + d];
+    if (half == 0 && t_chunk + n_chunk == q_start[s + 1]) {
+        const float m_end = ck.ends[z * 2] + fmaxf(m_start, ck.ends[z * 2 + 1]);
+        float* lev = level + (static_cast<size_t>(slots[s]) * in.heads + h) * (vdim + 1);
+        for (int col = tid; col <= vdim; col += NT) lev[col] = m_end;
+    }
+    chunk_gates(in, h, t_chunk, n_chunk, b_s, a_s, M_s, scratch);           // (its barriers also cover the staged rows)
 
     // the memory in front of the chunk: acc[j][rt] = S_start^T q
     f32x4 acc[NCT][4];
@@ -547,28 +669,18 @@ __global__ __launch_bounds__(NW * 64) void mlstm_chunk_read_kernel(MlstmInput in
     for (int j = 0; j < NCT; ++j)
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) acc[j][rt] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < ds; ++k) {
-        const int d0 = k * 32 + qd * 8;
+#pragma unroll
+    for (int k = 0; k < DS; ++k) {
         bf16x8 fq[4];
 #pragma unroll
-        for (int rt = 0; rt < 4; ++rt) fq[rt] = *reinterpret_cast<const bf16x8*>(q_l + (rt * 16 + r) * QS + d0);
+        for (int rt = 0; rt < 4; ++rt) fq[rt] = *reinterpret_cast<const bf16x8*>(q_l + (rt * 16 + r) * QS + k * 32 + qd * 8);
 #pragma unroll
-        for (int j = 0; j < NCT; ++j) {
-            const int ct = wave + NW * j;
-            if (ct >= nvt) continue;
-            bf16x8 fh, fl;
-#pragma unroll
-            for (int e = 0; e < 8; ++e) fh[e] = fl[e] = static_cast<bf16>(0.f);
-            if (d0 < dim) {
-                fh = *reinterpret_cast<const bf16x8*>(ck.s_hi + (z * vdim + ct * 16 + r) * dim + d0);
-                fl = *reinterpret_cast<const bf16x8*>(ck.s_lo + (z * vdim + ct * 16 + r) * dim + d0);
-            }
+        for (int j = 0; j < NCT; ++j)
 #pragma unroll
             for (int rt = 0; rt < 4; ++rt) {
-                acc[j][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fh, fq[rt], acc[j][rt], 0, 0, 0);
-                acc[j][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fl, fq[rt], acc[j][rt], 0, 0, 0);
+                acc[j][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(s_hi[j][k], fq[rt], acc[j][rt], 0, 0, 0);
+                acc[j][rt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(s_lo[j][k], fq[rt], acc[j][rt], 0, 0, 0);
             }
-        }
     }
     float M_row[4], start_w[4];                                             // of this lane's rows
 #pragma unroll
@@ -595,14 +707,18 @@ __global__ __launch_bounds__(NW * 64) void mlstm_chunk_read_kernel(MlstmInput in
     const float M_mine = M_row[rt_mine];
     float sum = 0.f;
     for (int key0 = 0; key0 <= row0; key0 += KB) {
-        const int count = min(KB, n_chunk - key0);
-        stage_rows(k_l, in.k_col, key0, count);
-        stage_values(key0, count);
-        __syncthreads();
+        // (the first keys are staged already; the next ones travel while these are worked through)
+        const bool more = key0 + KB <= row0;
+        float4 xk[QI], xv[VI][4];
+        if (more) {
+            load_rows(xk, in.k_col, key0 + KB, min(KB, n_chunk - key0 - KB));
+            load_values(xv, key0 + KB, min(KB, n_chunk - key0 - KB));
+        }
 #pragma unroll
         for (int kt = 0; kt < KT; ++kt) {
             f32x4 sc{0.f, 0.f, 0.f, 0.f};
-            for (int k = 0; k < ds; ++k) {
+#pragma unroll
+            for (int k = 0; k < DS; ++k) {
                 const int d0 = k * 32 + qd * 8;
                 const bf16x8 fk = *reinterpret_cast<const bf16x8*>(k_l + ((kt0 + kt) * 16 + r) * QS + d0);
                 const bf16x8 fq = *reinterpret_cast<const bf16x8*>(q_l + (rt_mine * 16 + r) * QS + d0);
@@ -643,7 +759,12 @@ __global__ __launch_bounds__(NW * 64) void mlstm_chunk_read_kernel(MlstmInput in
                 }
             }
         }
-        __syncthreads();                                    // (before the next keys take this block's place)
+        if (more) {
+            __syncthreads();                                // (before the next keys take this block's place)
+            put_rows(k_l, xk);
+            put_values(xv);
+            __syncthreads();
+        }
     }
     sum += __shfl_xor(sum, 16, kWave);
     sum += __shfl_xor(sum, 32, kWave);
@@ -743,6 +864,37 @@ extern "C" int llme_mlstm_finish(const float* o, const float* w, const float* g,
     return launch_status();
 }
 
+// A step of one row a request (row s is request s): the row through the memory and finished. out [T, ld_out] in out_dtype, the
+// gate's sums at g_col of p.
+extern "C" int llme_mlstm_single(const float* p, int ld, int q_col, int k_col, int v_col, int g_col, int i_col, int f_col, const float* bias,
+                                 float cap, float q_scale, int heads, int dim, int vdim, float* memory, float* level, const int* slots, int T,
+                                 const float* norm_w, float eps, float scale, void* out, int out_dtype, int ld_out, hipStream_t stream) {
+    if (T <= 0) return 0;
+    if (heads <= 0 || dim <= 0 || vdim <= 0 || !(cap > 0.f)) return kErrBadArgument;
+    if (dim > 256 || vdim > 8192) return kErrUnsupported;
+    const MlstmInput in = mlstm_input(p, ld, q_col, k_col, v_col, i_col, f_col, bias, cap, q_scale, heads, dim, vdim);
+    const bool vec = dim % 4 == 0 && ld % 4 == 0 && q_col % 4 == 0 && k_col % 4 == 0 && reinterpret_cast<uintptr_t>(p) % 16 == 0 &&
+                     reinterpret_cast<uintptr_t>(memory) % 16 == 0;
+    const size_t lds = static_cast<size_t>(vdim + 1) * 4;
+#define LLME_SINGLE_T(R, VEC, TO)                                                                                                    \
+    hipLaunchKernelGGL((mlstm_single_kernel<R, VEC, TO>), dim3(T, heads), dim3(1024), lds, stream, in, memory, level, slots, norm_w, \
+                       g_col, eps, scale, static_cast<TO*>(out), ld_out)
+#define LLME_SINGLE(R)                                                  \
+    do {                                                                \
+        if (vec && out_dtype == kF32) LLME_SINGLE_T(R, true, float);    \
+        else if (vec) LLME_SINGLE_T(R, true, bf16);                     \
+        else if (out_dtype == kF32) LLME_SINGLE_T(R, false, float);     \
+        else LLME_SINGLE_T(R, false, bf16);                             \
+    } while (0)
+    if (out_dtype != kF32 && out_dtype != kBF16) return kErrBadArgument;
+    if (dim <= 64) LLME_SINGLE(4);
+    else if (dim <= 128) LLME_SINGLE(8);
+    else LLME_SINGLE(16);
+#undef LLME_SINGLE
+#undef LLME_SINGLE_T
+    return launch_status();
+}
+
 extern "C" int llme_mlstm_chunk(void) { return kChunk; }
 
 // The chunked form: p as above with its rows and columns aligned to 16 bytes, dim a multiple of 8 and vdim of 16, both up
@@ -775,26 +927,32 @@ extern "C" int llme_mlstm_chunked(const float* p, int ld, int q_col, int k_col, 
     const int items = heads * (vdim + 1) * (dim / 4);
     hipLaunchKernelGGL(mlstm_chunk_carry_kernel, dim3((items + 255) / 256, n_seq), dim3(256), 0, stream, memory, level, q_start, slots, heads,
                        dim, vdim, ck);
-    hipLaunchKernelGGL(mlstm_chunk_level_kernel, dim3(heads, n_seq), dim3(256), 0, stream, level, q_start, slots, heads, vdim, ck);
-    const int DP = (dim + 31) / 32 * 32;
+    const int DP = dim <= 64 ? 64 : dim <= 128 ? 128 : 256;
     const int lds = 2 * (2 * 64 * (DP + 8) + vdim * 72 + 2 * 64 * 72);
     const dim3 read_grid(n_seq * n_chunks * 2, heads);
-#define LLME_READ(NW, NCT)                                                                                                          \
+#define LLME_READ_DS(NW, NCT, DS)                                                                                                          \
     do {                                                                                                                            \
         static bool attr_set = false;                                                                                               \
         if (!attr_set) {                                                                                                            \
-            const hipError_t err = hipFuncSetAttribute(reinterpret_cast<const void*>(&mlstm_chunk_read_kernel<NW, NCT>),           \
+            const hipError_t err = hipFuncSetAttribute(reinterpret_cast<const void*>(&mlstm_chunk_read_kernel<NW, NCT, DS>),           \
                                                        hipFuncAttributeMaxDynamicSharedMemorySize, 150 * 1024);                     \
             if (err != hipSuccess) return static_cast<int>(err);                                                                    \
             attr_set = true;                                                                                                        \
         }                                                                                                                           \
-        hipLaunchKernelGGL((mlstm_chunk_read_kernel<NW, NCT>), read_grid, dim3(NW * 64), lds, stream, in, q_start, n_chunks, ck,    \
+        hipLaunchKernelGGL((mlstm_chunk_read_kernel<NW, NCT, DS>), read_grid, dim3(NW * 64), lds, stream, in, q_start, n_chunks, slots, level, ck,    \
                            norm_w, g_col, eps, scale, static_cast<bf16*>(out), ld_out);                                             \
+    } while (0)
+#define LLME_READ(NW, NCT)                           \
+    do {                                             \
+        if (dim <= 64) LLME_READ_DS(NW, NCT, 2);     \
+        else if (dim <= 128) LLME_READ_DS(NW, NCT, 4); \
+        else LLME_READ_DS(NW, NCT, 8);               \
     } while (0)
     if (vdim <= 64) LLME_READ(4, 1);
     else if (vdim <= 128) LLME_READ(8, 1);
     else LLME_READ(8, 2);
 #undef LLME_READ
+#undef LLME_READ_DS
     return launch_status();
 }
 

@@ -13,17 +13,18 @@
 namespace llme {
 
 template <typename TW, typename TN, typename TO>
-__global__ __launch_bounds__(256) void norm_add_kernel(const float* __restrict__ y, const TW* __restrict__ w_post,
+__global__ __launch_bounds__(256) void norm_add_kernel(float* __restrict__ y, const TW* __restrict__ w_post,
                                                        float* __restrict__ h, const TN* __restrict__ w_next,
-                                                       TO* __restrict__ x_out, int H, float eps, float scale) {
+                                                       TO* __restrict__ x_out, int H, float eps, float scale, int clear) {
     extern __shared__ float row[];
     __shared__ float scratch[4];
     const int t = blockIdx.x;
-    const float* yr = y + static_cast<size_t>(t) * H;
+    float* yr = y + static_cast<size_t>(t) * H;
     float* hr = h + static_cast<size_t>(t) * H;
     float ss = 0.f;
     for (int i = threadIdx.x; i < H; i += 256) {
         const float v = yr[i];
+        if (clear) yr[i] = 0.f;
         row[i] = v;
         ss = fmaf(v, v, ss);
     }
@@ -71,12 +72,12 @@ template <> __device__ __forceinline__ void na_store4<bf16>(bf16* p, const float
 }
 
 template <typename TW, typename TN, typename TO, int NV>
-__global__ __launch_bounds__(256) void norm_add_vec_kernel(const float* __restrict__ y, const TW* __restrict__ w_post,
+__global__ __launch_bounds__(256) void norm_add_vec_kernel(float* __restrict__ y, const TW* __restrict__ w_post,
                                                            float* __restrict__ h, const TN* __restrict__ w_next,
-                                                           TO* __restrict__ x_out, int H, float eps, float scale) {
+                                                           TO* __restrict__ x_out, int H, float eps, float scale, int clear) {
     __shared__ float scratch[4];
     const int t = blockIdx.x;
-    const float* yr = y + static_cast<size_t>(t) * H;
+    float* yr = y + static_cast<size_t>(t) * H;
     float* hr = h + static_cast<size_t>(t) * H;
     float yv[NV][4], hv[NV][4], wv[NV][4], nv[NV][4];
 #pragma unroll
@@ -107,6 +108,7 @@ __global__ __launch_bounds__(256) void norm_add_vec_kernel(const float* __restri
             ss2 = fmaf(hv[k][e], hv[k][e], ss2);
         }
         if (i < H) na_store4(hr + i, hv[k]);
+        if (clear && i < H) *reinterpret_cast<float4*>(yr + i) = float4{0.f, 0.f, 0.f, 0.f};
     }
     if (x_out == nullptr) return;
     TO* xr = x_out + static_cast<size_t>(t) * H;
@@ -144,8 +146,9 @@ __global__ void soft_cap_kernel(float* __restrict__ x, size_t n, float cap) {
 
 using namespace llme;
 
-extern "C" int llme_norm_add(const float* y, const void* w_post, int w_dtype, float* h, const void* w_next,
-                             int wn_dtype, void* x_out, int xo_dtype, int T, int H, float eps, float scale, hipStream_t stream) {
+// clear: y is all zeros afterwards (for a product that adds its parts into it).
+extern "C" int llme_norm_add(float* y, const void* w_post, int w_dtype, float* h, const void* w_next,
+                             int wn_dtype, void* x_out, int xo_dtype, int T, int H, float eps, float scale, int clear, hipStream_t stream) {
     if (T <= 0) return 0;
     if (H <= 0 || H > 16000) return kErrUnsupported;
     const size_t lds = static_cast<size_t>(H) * sizeof(float);
@@ -155,7 +158,7 @@ extern "C" int llme_norm_add(const float* y, const void* w_post, int w_dtype, fl
     const int nv = !vec ? 0 : H <= 2048 ? 2 : H <= 4096 ? 4 : 8;
 #define LLME_NAV(TW, TN, TO, NV)                                                                          \
     hipLaunchKernelGGL((norm_add_vec_kernel<TW, TN, TO, NV>), dim3(T), dim3(256), 0, stream, y,           \
-                       static_cast<const TW*>(w_post), h, static_cast<const TN*>(w_next), static_cast<TO*>(x_out), H, eps, scale)
+                       static_cast<const TW*>(w_post), h, static_cast<const TN*>(w_next), static_cast<TO*>(x_out), H, eps, scale, clear)
 #define LLME_NA(TW, TN, TO)                                                                               \
     do {                                                                                                  \
         if (nv == 2) LLME_NAV(TW, TN, TO, 2);                                                             \
@@ -164,7 +167,7 @@ extern "C" int llme_norm_add(const float* y, const void* w_post, int w_dtype, fl
         else                                                                                              \
             hipLaunchKernelGGL((norm_add_kernel<TW, TN, TO>), dim3(T), dim3(256), lds, stream, y,         \
                                static_cast<const TW*>(w_post), h, static_cast<const TN*>(w_next),         \
-                               static_cast<TO*>(x_out), H, eps, scale);                                          \
+                               static_cast<TO*>(x_out), H, eps, scale, clear);                                          \
     } while (0)
     if (w_next == nullptr) {
         // nothing more, or the updated rows as they are in x_out's type

@@ -40,7 +40,9 @@ constexpr int kMaxHeadEntries = 256;
 // keys); gridDim.y groups share a token's heads. The angles of the token's position are made once per workgroup.
 // Rows of p: queries at column 0, keys at k_col, values at v_col (v_col < 0: a value head is the key head as
 // projected, before norm and rotation).
-template <typename TQ, typename TC, typename TW>
+// A wavefront asks for the entries of NB of its heads (and of their partners in the rotation) before it works on the first.
+// EPL: entries of a head that a lane holds (dk <= 64 EPL).
+template <typename TQ, typename TC, typename TW, int EPL>
 __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict__ p, int ld, int nq, int nk, int nv, int dk, int dv,
                                                          int k_col, int v_col, const TW* __restrict__ wq, const TW* __restrict__ wk,
                                                          int unit_norm, float eps, const float* __restrict__ inv_freq, int rot, int pairs,
@@ -48,7 +50,7 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict
                                                          const int* __restrict__ positions, const int* __restrict__ seq_idx,
                                                          const int* __restrict__ block_table, int max_blocks,
                                                          TQ* __restrict__ q_out, TC* __restrict__ k_cache, TC* __restrict__ v_cache,
-                                                         int page) {
+                                                         int page, int write_v) {
     __shared__ float cs_t[kMaxHeadEntries / 2], sn_t[kMaxHeadEntries / 2];
     const int t = blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -67,40 +69,110 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict
         cs_t[f] = cs;
     }
     __syncthreads();
-    for (int u = blockIdx.y * 4 + wave; u < nq + nk; u += 4 * gridDim.y) {
-        const bool is_q = u < nq;
-        const int head = is_q ? u : u - nq;
-        const float* hp = row + (is_q ? head * dk : k_col + head * dk);
-        const TW* w = is_q ? wq : wk;
-        float r = 1.f;
-        if (w != nullptr || unit_norm) {
-            float ss = 0.f;
-            for (int e = lane; e < dk; e += 64) ss = fmaf(hp[e], hp[e], ss);
-            r = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(dk) + eps);
+    // this lane's entries: whether they turn, with which partner, which way, the norms' weights
+    int partner[EPL];
+    float cs_l[EPL], sn_l[EPL], wq_l[EPL], wk_l[EPL], wq_p[EPL], wk_p[EPL];
+#pragma unroll
+    for (int i = 0; i < EPL; ++i) {
+        const int e = lane + 64 * i;
+        partner[i] = -1;
+        cs_l[i] = 1.f;
+        sn_l[i] = 0.f;
+        wq_l[i] = wk_l[i] = wq_p[i] = wk_p[i] = 1.f;
+        if (e >= dk) continue;
+        if (wq != nullptr) wq_l[i] = to_float(wq[e]);
+        if (wk != nullptr) wk_l[i] = to_float(wk[e]);
+        if (e < rot) {
+            const bool first = pairs ? (e & 1) == 0 : e < half;
+            const int f = pairs ? e >> 1 : (e < half ? e : e - half);
+            partner[i] = pairs ? e ^ 1 : (e < half ? e + half : e - half);
+            cs_l[i] = cs_t[f];
+            sn_l[i] = first ? -sn_t[f] : sn_t[f];           // v cos - other sin for the first of a pair, v cos + other sin for the second
+            if (wq != nullptr) wq_p[i] = to_float(wq[partner[i]]);
+            if (wk != nullptr) wk_p[i] = to_float(wk[partner[i]]);
         }
-        for (int e = lane; e < dk; e += 64) {
-            const float raw = hp[e];
-            float v = w != nullptr ? raw * r * to_float(w[e]) : raw * r;
-            if (e < rot) {
-                const bool first = pairs ? (e & 1) == 0 : e < half;
-                const int f = pairs ? e >> 1 : (e < half ? e : e - half);
-                const int pe = pairs ? e ^ 1 : (e < half ? e + half : e - half);
-                const float other = w != nullptr ? hp[pe] * r * to_float(w[pe]) : hp[pe] * r;
-                const float sn = sn_t[f], cs = cs_t[f];
-                v = first ? v * cs - other * sn : v * cs + other * sn;
+    }
+    constexpr int NB = EPL == 1 ? 4 : 2;
+    const int stride = 4 * gridDim.y;
+    for (int u0 = blockIdx.y * 4 + wave; u0 < nq + nk; u0 += NB * stride) {
+        float raw[NB][EPL], oth[NB][EPL];
+#pragma unroll
+        for (int b = 0; b < NB; ++b) {
+            const int u = u0 + b * stride;
+            const float* hp = row + (u < nq ? u * dk : k_col + (u - nq) * dk);
+#pragma unroll
+            for (int i = 0; i < EPL; ++i) {
+                const int e = lane + 64 * i;
+                const bool ok = u < nq + nk && e < dk;
+                raw[b][i] = ok ? hp[e] : 0.f;
+                oth[b][i] = ok && partner[i] >= 0 ? hp[partner[i]] : 0.f;
             }
-            if (is_q) {
-                q_out[(static_cast<size_t>(t) * nq + head) * dk + e] = from_float<TQ>(v * q_temp);
-            } else {
-                k_cache[((static_cast<size_t>(pg) * nk + head) * page + in_page) * dk + e] = from_float<TC>(v);
-                if (v_col < 0) v_cache[((static_cast<size_t>(pg) * nv + head) * dv + e) * page + in_page] = from_float<TC>(raw);
+        }
+#pragma unroll
+        for (int b = 0; b < NB; ++b) {
+            const int u = u0 + b * stride;
+            if (u >= nq + nk) break;
+            const bool is_q = u < nq;
+            const int head = is_q ? u : u - nq;
+            float r = 1.f;
+            if (unit_norm || (is_q ? wq : wk) != nullptr) {
+                float ss = 0.f;
+#pragma unroll
+                for (int i = 0; i < EPL; ++i) ss = fmaf(raw[b][i], raw[b][i], ss);
+                r = 1.0f / sqrtf(wave_sum(ss) / static_cast<float>(dk) + eps);
+            }
+#pragma unroll
+            for (int i = 0; i < EPL; ++i) {
+                const int e = lane + 64 * i;
+                if (e >= dk) continue;
+                float v = raw[b][i] * r * (is_q ? wq_l[i] : wk_l[i]);
+                if (e < rot) v = v * cs_l[i] + oth[b][i] * r * (is_q ? wq_p[i] : wk_p[i]) * sn_l[i];
+                if (is_q) {
+                    q_out[(static_cast<size_t>(t) * nq + head) * dk + e] = from_float<TQ>(v * q_temp);
+                } else {
+                    k_cache[((static_cast<size_t>(pg) * nk + head) * page + in_page) * dk + e] = from_float<TC>(v);
+                    if (v_col < 0) v_cache[((static_cast<size_t>(pg) * nv + head) * dv + e) * page + in_page] = from_float<TC>(raw[b][i]);
+                }
             }
         }
     }
-    if (v_col >= 0 && nv > 0) {
+    if (write_v && v_col >= 0 && nv > 0) {
         const float* vp = row + v_col;
         for (int e = blockIdx.y * 256 + threadIdx.x; e < nv * dv; e += 256 * gridDim.y)
             v_cache[((static_cast<size_t>(pg) * nv + e / dv) * dv + e % dv) * page + in_page] = from_float<TC>(vp[e]);
+    }
+}
+
+// The cache entries of a step's values where requests bring many rows: v_cache keeps a value entry's tokens side by side, so
+// eight tokens of a page (positions from a multiple of eight) are written as one piece. grid (pieces of the longest request,
+// requests, columns / 256); pieces that the request's rows fill in part are written entry by entry.
+template <typename TC>
+__global__ __launch_bounds__(256) void v_write_kernel(const float* __restrict__ p, int ld, int v_col, int nv, int dv,
+                                                      const int* __restrict__ positions, const int* __restrict__ q_start,
+                                                      const int* __restrict__ block_table, int max_blocks, TC* __restrict__ v_cache,
+                                                      int page) {
+    const int s = blockIdx.y;
+    const int e = blockIdx.z * 256 + threadIdx.x;
+    const int row0 = q_start[s], n = q_start[s + 1] - row0;
+    if (n <= 0 || e >= nv * dv) return;
+    const int ctx = positions[row0];
+    const int base = (ctx / 8 + blockIdx.x) * 8;            // the piece's first position
+    if (base >= ctx + n) return;
+    const int pg = block_table[static_cast<size_t>(s) * max_blocks + base / page];
+    TC* dst = v_cache + ((static_cast<size_t>(pg) * nv + e / dv) * dv + e % dv) * page + base % page;
+    const float* src = p + v_col + e;
+    const int lo = base < ctx ? ctx - base : 0, hi = base + 8 > ctx + n ? ctx + n - base : 8;
+    struct alignas(sizeof(TC) * 8) Piece { TC x[8]; };
+    Piece piece;
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+        if (j >= lo && j < hi) piece.x[j] = from_float<TC>(src[static_cast<size_t>(row0 + base + j - ctx) * ld]);
+    if (lo == 0 && hi == 8) {
+        *reinterpret_cast<Piece*>(dst) = piece;
+    } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+            if (j >= lo && j < hi) dst[j] = piece.x[j];
     }
 }
 
@@ -337,7 +409,8 @@ using namespace llme;
 extern "C" int llme_qk_prepare(const float* p, int ld, int nq, int nk, int nv, int dk, int dv, int k_col, int v_col,
                                const void* wq, const void* wk, int w_dtype, int unit_norm, float eps, const float* inv_freq, int rot,
                                int pairs, float qt_coef, int qt_every, const int* positions, const int* seq_idx, const int* block_table, int max_blocks, void* q_out,
-                               int q_dtype, void* k_cache, void* v_cache, int cache_dtype, int page, int T, hipStream_t stream) {
+                               int q_dtype, void* k_cache, void* v_cache, int cache_dtype, int page, int T, const int* q_start,
+                               int n_seq, int max_new, hipStream_t stream) {
     if (T <= 0) return 0;
     if (dk <= 0 || page <= 0 || rot < 0 || rot > dk || rot % 2 != 0 || qt_every < 0) return kErrBadArgument;
     if (nk > 0 && (dv <= 0 || nv <= 0 || nk % nv != 0 || k_cache == nullptr || v_cache == nullptr)) return kErrBadArgument;
@@ -349,17 +422,36 @@ extern "C" int llme_qk_prepare(const float* p, int ld, int nq, int nk, int nv, i
     // enough workgroups for the chip where the step has few tokens: up to a wavefront a head
     const int head_groups = (nq + nk + 3) / 4;
     const int want = (2048 + T - 1) / T;
+    // values of requests that bring many rows are written by a kernel of their own, eight tokens a piece
+    const int octets = q_start != nullptr && v_col >= 0 && nv > 0 && max_new >= 16 && page % 8 == 0 &&
+                               reinterpret_cast<uintptr_t>(v_cache) % 32 == 0 ? (max_new + 7) / 8 + 1 : 0;
     const dim3 grid(T, want < head_groups ? (want > 0 ? want : 1) : head_groups);
-#define LLME_PREP(TQ, TC, TW)                                                                                              \
-    hipLaunchKernelGGL((qk_prepare_kernel<TQ, TC, TW>), grid, dim3(256), 0, stream, p, ld, nq, nk, nv, dk, dv, k_col, v_col, \
+#define LLME_PREP(TQ, TC, TW)                     \
+    do {                                          \
+        if (dk <= 64) LLME_PREP_E(TQ, TC, TW, 1); \
+        else if (dk <= 128) LLME_PREP_E(TQ, TC, TW, 2); \
+        else LLME_PREP_E(TQ, TC, TW, 4);          \
+    } while (0)
+#define LLME_PREP_E(TQ, TC, TW, EPL)                                                                                              \
+    hipLaunchKernelGGL((qk_prepare_kernel<TQ, TC, TW, EPL>), grid, dim3(256), 0, stream, p, ld, nq, nk, nv, dk, dv, k_col, v_col, \
                        static_cast<const TW*>(wq), static_cast<const TW*>(wk), unit_norm, eps, inv_freq, rot, pairs, qt_coef, qt_every, positions, seq_idx, \
-                       block_table, max_blocks, static_cast<TQ*>(q_out), static_cast<TC*>(k_cache), static_cast<TC*>(v_cache), page)
+                       block_table, max_blocks, static_cast<TQ*>(q_out), static_cast<TC*>(k_cache), static_cast<TC*>(v_cache), page, octets == 0)
     if (q_dtype != cache_dtype) return kErrBadArgument;
     if (q_dtype == kF32 && w_dtype == kF32) LLME_PREP(float, float, float);
     else if (q_dtype == kBF16 && w_dtype == kF32) LLME_PREP(bf16, bf16, float);
     else if (q_dtype == kBF16 && w_dtype == kBF16) LLME_PREP(bf16, bf16, bf16);
     else return kErrBadArgument;
 #undef LLME_PREP
+#undef LLME_PREP_E
+    if (octets > 0) {
+        const dim3 vgrid(octets, n_seq, (nv * dv + 255) / 256);
+        if (cache_dtype == kF32)
+            hipLaunchKernelGGL((v_write_kernel<float>), vgrid, dim3(256), 0, stream, p, ld, v_col, nv, dv, positions, q_start, block_table,
+                               max_blocks, static_cast<float*>(v_cache), page);
+        else
+            hipLaunchKernelGGL((v_write_kernel<bf16>), vgrid, dim3(256), 0, stream, p, ld, v_col, nv, dv, positions, q_start, block_table,
+                               max_blocks, static_cast<bf16*>(v_cache), page);
+    }
     return launch_status();
 }
 

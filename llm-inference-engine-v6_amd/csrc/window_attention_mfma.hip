@@ -360,7 +360,10 @@ __global__ __launch_bounds__(256, 4) void window_attention_mfma_shared_kernel(Wi
     const int vh = kh / a.maps, map = kh % a.maps;
     const int row0 = a.q_start[s];
     const int rows_total = (a.q_start[s + 1] - row0) * a.per_value_head;
-    const int RW = blockIdx.x * 64;                         // the workgroup's first row
+    // Later rows see more keys (up to a window's or a chunk's length). Compute units are dealt workgroups at fixed distances
+    // of (x, y), so every other y takes its rows from the end: a unit's workgroups are then long and short ones.
+    const int bx = ((blockIdx.y ^ (blockIdx.y >> 1)) & 1) ? gridDim.x - 1 - blockIdx.x : blockIdx.x;
+    const int RW = bx * 64;                                 // the workgroup's first row
     if (RW >= rows_total) return;                           // (the whole workgroup)
     const int R0 = RW + wave * 16;
     const bool active = R0 < rows_total;

@@ -15,7 +15,7 @@ LATENT_MAX_ROW, LATENT_MAX_RANK = 1024, 512         # the plain attention kernel
 MOE_MAX_EXPERTS = 1024
 MOE_TILE = 16
 
-declare("llme_norm_add", [_vp, _vp, _i, _vp, _vp, _i, _vp, _i, _i, _i, _f, _f, _vp])
+declare("llme_norm_add", [_vp, _vp, _i, _vp, _vp, _i, _vp, _i, _i, _i, _f, _f, _i, _vp])
 declare("llme_soft_cap_f32", [_vp, _z, _f, _vp])
 declare("llme_scale_f32", [_vp, _z, _f, _vp])
 declare("llme_latent_prepare", [_vp, _i, _i, _i, _i, _i, _vp, _vp, _i, _vp, _f, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _f, _vp])
@@ -30,9 +30,9 @@ declare("llme_moe_combine", [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp])
 
 # --- sandwich norm ---------------------------------------------------------------------
 def norm_add(y: torch.Tensor, w_post: torch.Tensor, h: torch.Tensor, eps: float, w_next: torch.Tensor | None = None,
-             x_out: torch.Tensor | None = None, scale: float = 1.0) -> None:
+             x_out: torch.Tensor | None = None, scale: float = 1.0, clear: bool = False) -> None:
     """h += scale * (w_post * y / rms(y)); with w_next also x_out = w_next * h / rms(h) of the updated rows; with x_out and no
-    w_next, x_out = the updated rows as they are, in x_out's type. y, h [T, H] 32-bit; the weights multiply as they are."""
+    w_next, x_out = the updated rows as they are, in x_out's type. clear: y is all zeros afterwards. y, h [T, H] 32-bit; the weights multiply as they are."""
     require(y, "y", torch.float32, (None, None))
     T, H = y.shape
     require(h, "h", torch.float32, (T, H))
@@ -43,7 +43,7 @@ def norm_add(y: torch.Tensor, w_post: torch.Tensor, h: torch.Tensor, eps: float,
         require(x_out, "x_out", _FLOATS, (T, H))
     check(entry("llme_norm_add")(ptr(y), ptr(w_post), code(w_post.dtype), ptr(h), ptr(w_next),
                                  code(w_next.dtype) if w_next is not None else 0, ptr(x_out),
-                                 code(x_out.dtype) if x_out is not None else 0, T, H, float(eps), float(scale), stream()), "norm_add")
+                                 code(x_out.dtype) if x_out is not None else 0, T, H, float(eps), float(scale), 1 if clear else 0, stream()), "norm_add")
 
 
 def scale_(x: torch.Tensor, s: float) -> None:

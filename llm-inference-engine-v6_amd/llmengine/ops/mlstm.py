@@ -12,13 +12,16 @@ from .recurrent import _cols
 
 _vp, _i, _f = ctypes.c_void_p, ctypes.c_int, ctypes.c_float
 _FLOATS = (torch.float32, torch.bfloat16)
+MAX_VDIM_SINGLE = 8192          # value entries of a head that the kernel for steps of single rows holds
 MAX_DIM = 256                   # key channels of a head that the kernels hold
 CHUNK_FROM = 48                 # rows a request brings from which a bfloat16 model's chunked kernels take it (smaller: the walk)
 CHUNK_BYTES = 4 << 30           # the most scratch memory the chunked form may take
 NEVER = 1 << 30
+SINGLE_ROWS = True              # steps of one row a request have a kernel of their own (False: the walk; tests, measurements)
 
 declare("llme_mlstm_walk", [_vp, _i, _i, _i, _i, _i, _i, _vp, _f, _f, _i, _i, _i, _vp, _vp, _vp, _vp, _vp, _i, _i, _vp])
 declare("llme_mlstm_finish", [_vp, _vp, _vp, _i, _vp, _i, _i, _i, _i, _i, _f, _f, _vp, _vp, _i, _vp])
+declare("llme_mlstm_single", [_vp, _i, _i, _i, _i, _i, _i, _i, _vp, _f, _f, _i, _i, _i, _vp, _vp, _vp, _i, _vp, _f, _f, _vp, _i, _i, _vp])
 declare("llme_mlstm_chunk", [])
 declare("llme_mlstm_chunked", [_vp, _i, _i, _i, _i, _i, _i, _i, _vp, _f, _f, _i, _i, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _vp, _vp, _vp,
                                _vp, _vp, _vp, _vp, _f, _f, _vp, _i, _vp])
@@ -68,6 +71,11 @@ def mlstm(p: torch.Tensor, cols: MlstmColumns, gate_bias: torch.Tensor, cap: flo
     if T != step.num_tokens:
         raise KernelError("mlstm: one row per token of the step")
     q_scale = float(dim) ** -0.5
+    if T == step.num_seqs and vdim <= MAX_VDIM_SINGLE and SINGLE_ROWS:
+        check(entry("llme_mlstm_single")(ptr(p), ld, cols.q, cols.k, cols.v, cols.g, cols.i, cols.f, ptr(gate_bias), float(cap), q_scale,
+                                         heads, dim, vdim, ptr(memory), ptr(level), ptr(step.slots), T, ptr(norm_w), float(eps),
+                                         float(scale), ptr(out), code(out.dtype), ld_out, stream()), "mlstm_single")
+        return
     limit = CHUNK_FROM if chunk_from is None else int(chunk_from)
     longest = max(step.new_lens)
     if longest >= limit and chunked_fits(p, cols, out, dim, vdim):

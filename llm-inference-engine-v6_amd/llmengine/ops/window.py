@@ -17,7 +17,7 @@ FINISH_MODES = {"plain": 0, "gate": 1, "difference": 2, "head_gate": 3}
 BIAS_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "swish_clamped": 3}
 
 declare("llme_qk_prepare", [_vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _i, _i, _f, _vp, _i, _i, _f, _i, _vp, _vp, _vp, _i, _vp, _i, _vp,
-                            _vp, _i, _i, _i, _vp])
+                            _vp, _i, _i, _i, _vp, _i, _i, _vp])
 declare("llme_window_attention", [_vp, _i, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i, _i, _vp,
                                   _vp])
 declare("llme_window_attention_finish", [_vp, _vp, _i, _i, _i, _i, _i, _i, _vp, _i, _f, _f, _f, _vp, _vp, _i, _i, _vp])
@@ -85,7 +85,7 @@ def qk_prepare(p: torch.Tensor, step, block_table: torch.Tensor | None, q_out: t
                                    1 if pairs == "neighbours" else 0, coef, every,
                                    ptr(step.positions), ptr(step.seq_idx), ptr(block_table) if nk else None,
                                    block_table.shape[1] if nk else 0, ptr(q_out), code(q_out.dtype), ptr(k_cache), ptr(v_cache),
-                                   code(q_out.dtype), page, T, stream()), "qk_prepare")
+                                   code(q_out.dtype), page, T, ptr(step.q_start), step.num_seqs, max(step.new_lens), stream()), "qk_prepare")
 
 
 declare("llme_window_attention_mfma", [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i, _i,

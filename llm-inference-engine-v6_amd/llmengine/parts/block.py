@@ -146,6 +146,7 @@ class OutputNormBlock(Block):
     the norm behind it, the sum into the stream and the copy of the updated rows that the next sublayer reads (this
     block's feed-forward, or the mixer of the block behind) are one kernel."""
     graph_safe = True
+    ADDED_ROWS = 64             # steps of up to this many rows add the parts of a sublayer's last product
 
     def __init__(self, mixer: Mixer, feed_forward: FeedForward | None, mixer_norm: Norm, ffn_norm: Norm | None,
                  names: dict | None = None, residual_scale: float = 1.0):
@@ -165,30 +166,39 @@ class OutputNormBlock(Block):
             out.update({n["ffn_norm"]: self.ffn_norm, n["feed_forward"]: self.feed_forward})
         return out
 
-    def _join(self, y, post: Norm, h, x) -> None:
+    def _join(self, y, post: Norm, h, x, clear: bool) -> None:
         """h += c post(y), and x = the updated rows where x is another buffer than the stream."""
         rms = post.fused_rms()
         if rms is None:
             raise NotImplementedError("output-norm blocks take norms of the plain RMS formula behind their sublayers")
-        ops.norm_add(y, rms[0], h, rms[1], None, x if x is not h else None, self.residual_scale)
+        ops.norm_add(y, rms[0], h, rms[1], None, x if x is not h else None, self.residual_scale, clear)
 
     def forward(self, h, step, cache, write_cache=True):
         T, H = h.shape
-        y = step.buffer("block.sublayer", (T, H), torch.float32)
+        # few rows: a sublayer's last product is cut over k and its parts are added (atomics) into a buffer of zeros, which
+        # the norm behind it leaves as zeros again; otherwise it is stored
+        add = T <= self.ADDED_ROWS and not step.fixed_order and step.act_dtype == torch.bfloat16 and H % 4 == 0
+        if add:
+            y = step.buffer("block.sublayer_sum", (T, H), torch.float32)
+            if not step.extra.get("block.sublayer_sum is clear"):
+                ops.clear(y)
+                step.extra["block.sublayer_sum is clear"] = True
+        else:
+            y = step.buffer("block.sublayer", (T, H), torch.float32)
         if step.act_dtype == torch.float32:
             x = h                           # (the sublayers read the 32-bit stream as it lies)
         else:
             x = step.buffer("block.stream_copy", (T, H), step.act_dtype)
             if step.extra.pop("block.stream_copy is for", None) != id(self):
                 ops.copy_cols(h, x)
-        self.mixer.forward(x, step, cache, y, False, write_cache)
+        self.mixer.forward(x, step, cache, y, add, write_cache)
         hand_on = isinstance(self.next_block, OutputNormBlock) and x is not h
         if self.feed_forward is None:
-            self._join(y, self.mixer_norm, h, x if hand_on else h)
+            self._join(y, self.mixer_norm, h, x if hand_on else h, add)
         else:
-            self._join(y, self.mixer_norm, h, x)
-            self.feed_forward.forward(x, step, y, False)
-            self._join(y, self.ffn_norm, h, x if hand_on else h)
+            self._join(y, self.mixer_norm, h, x, add)
+            self.feed_forward.forward(x, step, y, add)
+            self._join(y, self.ffn_norm, h, x if hand_on else h, add)
         if hand_on:
             step.extra["block.stream_copy is for"] = id(self.next_block)
 
