@@ -236,8 +236,9 @@ class _Step:
     (2, 32, 48, 6.0, [300, 1, 64, 130]), (3, 128, 256, 15.0, [257]), (1, 256, 64, 4.0, [128, 5, 129]), (2, 40, 112, 10.0, [48, 47, 200]),
     (4, 64, 64, 30.0, [1, 1, 500, 1]), (2, 8, 16, 2.0, [640]), (1, 200, 240, 8.0, [127, 1, 128]), (3, 56, 32, 5.0, [1, 2, 3, 4, 1]),
     (2, 128, 256, 9.0, [1, 1, 1]), (5, 17, 33, 9.0, [1, 1]), (1, 256, 300, 9.0, [1, 1, 1, 1])])
-def test_the_memory_kernels_against_the_recurrence(heads, dim, vdim, cap, lens):
-    """The memory's operation on rows, states and levels drawn at random: both forms against the recurrence in float64 (rows
+def test_the_memory_kernels_against_the_recurrence(heads, dim, vdim, cap, lens, monkeypatch):
+    """The memory's operation on rows, states and levels drawn at random: every form (the walk, chunks, the kernel for steps
+    of single rows) against the recurrence in float64 (rows
     and states afterwards), requests of every length side by side, slots in any order, the others untouched."""
     from llmengine import ops
     g = torch.Generator().manual_seed(heads * 1000 + dim + vdim)
@@ -273,7 +274,9 @@ def test_the_memory_kernels_against_the_recurrence(heads, dim, vdim, cap, lens):
         want_lev[slots[s]] = state[2][:, None]
         at += n
     rel = lambda a, b: float((a.double().cpu() - b).abs().max() / b.abs().max())
-    for dtype, chunk_from in ((torch.float32, None), (torch.bfloat16, ops.mlstm.NEVER), (torch.bfloat16, 48), (torch.bfloat16, 2)):
+    for dtype, chunk_from, single in ((torch.float32, None, True), (torch.float32, None, False), (torch.bfloat16, ops.mlstm.NEVER, False),
+                                      (torch.bfloat16, 48, True), (torch.bfloat16, 2, False)):
+        monkeypatch.setattr(ops.mlstm, "SINGLE_ROWS", single)
         mem, lev = memory.cuda(), level.cuda()
         # (the result is a column range of a wider buffer, as beside another mixer)
         wide = torch.full((T, hv + 32), 7.0, dtype=dtype, device="cuda")
@@ -511,6 +514,37 @@ def test_long_decoding_in_bfloat16_on_the_matrix_cores(tmp_path):
     got = replay.run_trace(engine, engine.new_cache(16, 16, 2), replay.tail_one_by_one({"r": ids}, tail=190))
     assert _as_rounding(got, whole, honest) and _as_rounding(got, ref, honest)
     assert engine.runner.graph_replays >= 189
+
+
+@pytest.mark.parametrize("cfg_name", ["MIXED", "ALIGNED"])
+def test_sums_that_are_split_as_serving_does(tmp_path, cfg_name):
+    """Without the promise of one order of sums, steps of few rows cut a sublayer's last product over k and add the parts
+    into a buffer that the norm behind it leaves as zeros; whole prompts, portions and recorded steps follow one another."""
+    from llmengine import Engine
+    cfg = getattr(lm, cfg_name)
+    folder, weights = lm.write_model(tmp_path, cfg, 19)
+    engine = Engine(folder, "bf16")
+    V = cfg["vocab"]
+    requests = {"a": _tokens(130, V, 1), "b": _tokens(70, V, 2), "c": _tokens(5, V, 3)}
+    ref = _reference(cfg, weights, requests)
+    honest = _honest(cfg, weights, requests, ref)
+    for steps in (replay.tail_one_by_one(requests, tail=30), replay.whole(requests), replay.mixed(requests, max_live=3, sizes=(70, 3, 24, 2), seed=4),
+                  replay.portions(requests, sizes=(64, 65, 2))):
+        got = replay.run_trace(engine, _pool(engine, steps, 16, 3), steps)
+        assert _covered(got, requests) and _as_rounding(got, ref, honest)
+
+
+@pytest.mark.parametrize("page", [4, 12, 24, 64])
+def test_pages_of_other_sizes(tmp_path, page):
+    """Values are written eight tokens a piece where pages hold whole pieces, and token by token otherwise."""
+    cfg = lm.config([lm.chunked(chunk=30, sharp=2.0, ff=None), lm.chunked(heads=2, kv_heads=1, dim=16, vdim=20, chunk=0, ff=12)])
+    engine, weights = _engine(tmp_path, cfg, 25, "fp32")
+    V = cfg["vocab"]
+    requests = {"a": _tokens(150, V, 1), "b": _tokens(39, V, 2)}
+    ref = _reference(cfg, weights, requests)
+    for steps in (replay.whole(requests), replay.portions(requests, sizes=(17, 31, 2, 50)), replay.mixed(requests, max_live=2, sizes=(40, 3, 21), seed=1)):
+        got = replay.run_trace(engine, _pool(engine, steps, page, 2), steps)
+        assert _covered(got, requests) and _worst(got, ref) < F32_TOL
 
 
 def test_several_requests_decode_together_over_the_chunks_edges(tmp_path):
