@@ -35,6 +35,20 @@ __device__ __forceinline__ float wave_max(float v) {
     return v;
 }
 
+// The sum over each group of 8 or 16 neighbouring lanes, in every lane of the group, by data-parallel-primitive moves
+// inside the vector unit (a shuffle through LDS would put three trips to LDS into every step of the recurrence):
+// neighbours in a quad, the quad's other pair, then the mirror image in the half row of 8.
+template <int LANES>
+__device__ __forceinline__ float sum_of_lanes(float v) {
+    static_assert(LANES == 8 || LANES == 16, "groups of 8 or 16 lanes");
+    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true));     // quad_perm [1, 0, 3, 2]
+    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, true));     // quad_perm [2, 3, 0, 1]
+    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x141, 0xF, 0xF, true));    // row_half_mirror
+    if (LANES == 16)                                                                                                // and the row of 16's mirror image
+        v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x140, 0xF, 0xF, true));
+    return v;
+}
+
 // Sum over a whole workgroup of `nwaves` wavefronts; `scratch` holds >= nwaves floats.
 // Every thread gets the result. Contains two barriers.
 __device__ __forceinline__ float block_sum(float v, float* scratch, int nwaves) {

@@ -41,18 +41,6 @@ struct MlstmInput {
 __device__ __forceinline__ float capped_gate(float z, float cap) { return cap * tanhf(z / cap); }
 __device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
 
-// The sum over each group of 8 or 16 neighbouring lanes, in every lane of the group, by moves inside the vector unit.
-template <int LANES>
-__device__ __forceinline__ float sum_of_group(float v) {
-    static_assert(LANES == 8 || LANES == 16, "groups of 8 or 16 lanes");
-    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true));     // quad_perm [1, 0, 3, 2]
-    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, true));     // quad_perm [2, 3, 0, 1]
-    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x141, 0xF, 0xF, true));    // row_half_mirror
-    if (LANES == 16)
-        v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x140, 0xF, 0xF, true));  // row_mirror
-    return v;
-}
-
 // ---------------------------------------------------------------------------------------------------------------
 // The walk. LPC lanes share a column (lane l holds the R key channels l R ..), a workgroup owns 256 / LPC columns of one
 // head of one request. Rows come through LDS in blocks of eight (k, q, the columns' values, the two log gates, which are
@@ -150,7 +138,7 @@ __global__ __launch_bounds__(256) void mlstm_walk_kernel(MlstmInput in, float* _
                 reads[0] = fmaf(m[i], q2.x, reads[0]);
                 reads[1] = fmaf(m[i + 1], q2.y, reads[1]);
             }
-            const float read = sum_of_group<LPC>(reads[0] + reads[1]) * in.q_scale;
+            const float read = sum_of_lanes<LPC>(reads[0] + reads[1]) * in.q_scale;
             if (live && l == 0) {
                 float* orow = o + (static_cast<size_t>(t0 + tt) * in.heads + h) * (in.vdim + 2);
                 orow[col] = read;
@@ -262,7 +250,7 @@ __global__ __launch_bounds__(1024) void mlstm_single_kernel(MlstmInput in, float
                 for (int i = 0; i < R; ++i)
                     if (l * R + i < dim) M[i] = m[u][i];
             }
-            const float read = sum_of_group<16>(reads[0] + reads[1]) * in.q_scale;
+            const float read = sum_of_lanes<16>(reads[0] + reads[1]) * in.q_scale;
             if (l == 0) read_s[c] = read;
         }
     }
@@ -475,7 +463,7 @@ __global__ __launch_bounds__(256) void mlstm_chunk_add_kernel(MlstmInput in, con
             const int d = ((tid + 256 * i) >> 3) * 4;
 #pragma unroll
             for (int e = 0; e < 4; ++e) {
-                const float v = sum_of_group<8>(z_acc[i][e]);       // the pieces of the same channels: eight neighbouring lanes
+                const float v = sum_of_lanes<8>(z_acc[i][e]);       // the pieces of the same channels: eight neighbouring lanes
                 if ((lane & 7) == 0 && d + e < dim) add[static_cast<size_t>(vdim) * dim + d + e] = v;
             }
         }

@@ -345,20 +345,6 @@ __global__ __launch_bounds__(256) void sigmoid_decay_kernel(const float* __restr
 // memory while the current one is worked through, so that a step waits for LDS only.
 constexpr int kDeltaRows = 8, kDeltaFetch = 28;
 
-// The sum over each group of 8 or 16 neighbouring lanes, in every lane of the group, by data-parallel-primitive moves
-// inside the vector unit (a shuffle through LDS would put three trips to LDS into every step of the recurrence):
-// neighbours in a quad, the quad's other pair, then the mirror image in the half row of 8.
-template <int LANES>
-__device__ __forceinline__ float sum_of_lanes(float v) {
-    static_assert(LANES == 8 || LANES == 16, "groups of 8 or 16 lanes");
-    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0xB1, 0xF, 0xF, true));     // quad_perm [1, 0, 3, 2]
-    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x4E, 0xF, 0xF, true));     // quad_perm [2, 3, 0, 1]
-    v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x141, 0xF, 0xF, true));    // row_half_mirror
-    if (LANES == 16)                                                                                                // and the row of 16's mirror image
-        v += __builtin_bit_cast(float, __builtin_amdgcn_mov_dpp(__builtin_bit_cast(int, v), 0x140, 0xF, 0xF, true));
-    return v;
-}
-
 // DELTA false is the plain linear rule (gated linear attention): nothing is read back before the write,
 //   M <- g * M;  M <- M + k v^T;  o = M^T q,
 // and beta is not looked at. Every read is multiplied by o_scale (a scale on the queries).
