@@ -14,7 +14,9 @@
 //
 // Rotation: of a part's r entries the first rd are rotated, the rest pass unchanged; entries (2i, 2i + 1) turn by angle = position * freq[i], a 32-bit product; cos and sin are
 // multiplied by `mag` (1 without frequency scaling). A token at position p sees keys lo .. p of its own
-// request, lo = 0 or p - window + 1.
+// request, lo = 0 or p - window + 1. `sinks` (one number a head, or null): the softmax's denominator also holds
+// e^(sink_h), a key without a value; `gate` ([T, ld_gate] 32-bit, one number a head, or null): a head's sum is
+// multiplied by sigmoid(gate) (a factor of the whole sum, so the value map may follow it).
 //
 //   cache       [pages, page, D]; key t of request s lies in page block_table[s][t / page] at row t % page
 #include "common.h"
@@ -141,7 +143,7 @@ template <typename TQ, typename TC, int NW>
 __global__ __launch_bounds__(NW * 64) void latent_attention_kernel(
     const TQ* __restrict__ qp, const TC* __restrict__ cache, TQ* __restrict__ out, const int* __restrict__ positions,
     const int* __restrict__ seq_idx, const int* __restrict__ block_table, int max_blocks, int n, int R, int D, int page,
-    float scale, int window) {
+    float scale, int window, const float* __restrict__ sinks, const float* __restrict__ gate, int ld_gate) {
     constexpr int PER_LANE = kLatMaxR / kWave;
     __shared__ float qs[kLatMaxD];
     __shared__ float join_m[NW], join_l[NW];
@@ -208,8 +210,16 @@ __global__ __launch_bounds__(NW * 64) void latent_attention_kernel(
 #pragma unroll
             for (int i = 0; i < PER_LANE; ++i) acc[i] += f * join_acc[w][lane + i * kWave];
         }
+        m = mx;
     }
-    const float inv = 1.0f / l;
+    float inv = 1.0f / l;
+    if (sinks != nullptr) {                     // the sink joins like one more key whose value is nothing
+        const float sk = sinks[h];
+        const float top = fmaxf(m, sk);
+        const float f = expf(m - top);
+        inv = f / fmaf(l, f, expf(sk - top));
+    }
+    if (gate != nullptr) inv /= 1.0f + expf(-gate[static_cast<size_t>(t) * ld_gate + h]);
     TQ* orow = out + (static_cast<size_t>(t) * n + h) * R;
 #pragma unroll
     for (int i = 0; i < PER_LANE; ++i) {
@@ -278,9 +288,10 @@ extern "C" int llme_head_gemm(const void* a, int a_dtype, long lda, long sa, con
 
 extern "C" int llme_latent_attention(const void* qp, int q_dtype, const void* cache, int cache_dtype, void* out,
                                      const int* positions, const int* seq_idx, const int* block_table, int max_blocks,
-                                     int T, int n, int R, int D, int page, float scale, int window, hipStream_t stream) {
+                                     int T, int n, int R, int D, int page, float scale, int window, const float* sinks, const float* gate,
+                                     int ld_gate, hipStream_t stream) {
     if (T <= 0) return 0;
-    if (n <= 0 || R <= 0 || D < R || page <= 0) return kErrBadArgument;
+    if (n <= 0 || R <= 0 || D < R || page <= 0 || (gate != nullptr && ld_gate < n)) return kErrBadArgument;
     if (D > kLatMaxD || R > kLatMaxR || n > 65535) return kErrUnsupported;
     const dim3 grid(T, n);
     const bool few = static_cast<long>(T) * n < 4096;
@@ -289,11 +300,11 @@ extern "C" int llme_latent_attention(const void* qp, int q_dtype, const void* ca
         if (few)                                                                                              \
             hipLaunchKernelGGL((latent_attention_kernel<TQ, TC, 8>), grid, dim3(8 * 64), 0, stream,           \
                                static_cast<const TQ*>(qp), static_cast<const TC*>(cache), static_cast<TQ*>(out), \
-                               positions, seq_idx, block_table, max_blocks, n, R, D, page, scale, window);    \
+                               positions, seq_idx, block_table, max_blocks, n, R, D, page, scale, window, sinks, gate, ld_gate);    \
         else                                                                                                  \
             hipLaunchKernelGGL((latent_attention_kernel<TQ, TC, 1>), grid, dim3(64), 0, stream,               \
                                static_cast<const TQ*>(qp), static_cast<const TC*>(cache), static_cast<TQ*>(out), \
-                               positions, seq_idx, block_table, max_blocks, n, R, D, page, scale, window);    \
+                               positions, seq_idx, block_table, max_blocks, n, R, D, page, scale, window, sinks, gate, ld_gate);    \
     } while (0)
     if (q_dtype == kF32 && cache_dtype == kF32) LLME_LA(float, float);
     else if (q_dtype == kBF16 && cache_dtype == kBF16) LLME_LA(bf16, bf16);

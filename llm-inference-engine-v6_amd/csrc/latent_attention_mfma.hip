@@ -17,7 +17,11 @@
 // weights' sums go to a workspace and latent_join adds them in a fixed order.
 //
 // Softmax: running maximum m and sum l per row in units of log2; the sum adds the weights as rounded to
-// bfloat16, which is what the second product sees.
+// bfloat16, which is what the second product sees. A sink (one number a head: e^(sink) joins the sum, nothing the
+// values) and a sigmoid gate of one number a head enter where a row is divided by its sum: here with one run of keys,
+// in latent_join otherwise.
+//
+// Rows whose length is no multiple of 32 are staged with zeros behind them.
 //
 //   qa [.., R], qr [.., r]   a pair's rows at (token * q_ts + head * q_hs) * R resp. * r
 //   out [.., R]              at (token * o_ts + head * o_hs) * R
@@ -36,8 +40,9 @@ constexpr float kLatNoMax = -1.0e30f;
 constexpr int kVtStride = 40;           // elements of a transposed row: 32 keys + 8 (80 bytes: 8-byte reads without conflicts)
 
 __host__ __device__ inline int lat_k_stride(int D) {
-    // elements of a staged row: its bytes are 32 more than a multiple of 128, so that 16-byte operand reads run at full rate
-    const int bytes = D * 2;
+    // elements of a staged row (whole chunks of 32 entries): its bytes are 32 more than a multiple of 128, so that 16-byte
+    // operand reads run at full rate
+    const int bytes = (D + 31) / 32 * 64;
     return (bytes + ((32 - bytes % 128) + 128) % 128) / 2;
 }
 
@@ -54,12 +59,30 @@ struct LatentArgs {
     int max_blocks, T, n, R, r, page, window, nsplit;
     long q_ts, q_hs, o_ts, o_hs;
     float scale_log2;
+    const float* sinks;         // [n] or null
+    const float* gate;          // [T, ld_gate] or null
+    int ld_gate;
 };
+
+constexpr float kLog2E = 1.4426950408889634f;
+
+// What a row's weighted values are multiplied by: 2^(m - M) / (its sum), the sink in M and in the sum, times its gate.
+__device__ __forceinline__ float lat_row_factor(float m, float l, int tok, int h, const float* sinks, const float* gate, int ld_gate) {
+    float f = 1.0f / l;
+    if (sinks != nullptr) {
+        const float sk = sinks[h] * kLog2E;
+        const float top = fmaxf(m, sk);
+        const float scale = __builtin_amdgcn_exp2f(m - top);
+        f = scale / fmaf(l, scale, __builtin_amdgcn_exp2f(sk - top));
+    }
+    if (gate != nullptr) f /= 1.0f + expf(-gate[static_cast<size_t>(tok) * ld_gate + h]);
+    return f;
+}
 
 template <int DC, int RC>       // 32-entry chunks of a row, 16-entry chunks of the latent: the most this instance holds
 __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(LatentArgs a) {
     extern __shared__ __align__(16) unsigned char lds_raw[];
-    const int D = a.R + a.r, dc = D / 32, rc = a.R / 16;
+    const int D = a.R + a.r, dc = (D + 31) / 32, rc = a.R / 16;
     const int ks = lat_k_stride(D);
     bf16* Ks = reinterpret_cast<bf16*>(lds_raw);                    // [32][ks]
     bf16* Vt = Ks + 32 * ks;                                        // [R][kVtStride]
@@ -100,7 +123,7 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(LatentArgs a
             const int d = c * 32 + g * 8;
 #pragma unroll
             for (int e = 0; e < 8; ++e) qf[c][e] = static_cast<__bf16>(0.f);
-            if (c < dc && row_ok)
+            if (d < D && row_ok)
                 qf[c] = d < a.R ? *reinterpret_cast<const bf16x8*>(qa_row + d) : *reinterpret_cast<const bf16x8*>(qr_row + d - a.R);
         }
     }
@@ -139,6 +162,8 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(LatentArgs a
         }
     };
 
+    // (entries behind the rows' last, up to whole chunks: zeros, written once)
+    for (int i = tid; i < 32 * (dc * 32 - D); i += 256) Ks[(i % 32) * ks + D + i / 32] = static_cast<bf16>(0.f);
     if (b_begin < b_end) fetch(b_begin);
     for (int b = b_begin; b < b_end; ++b) {
         __syncthreads();                    // everybody has read the block before
@@ -209,6 +234,7 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(LatentArgs a
     // a row's sum over the four lanes that hold its keys
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);
+    const float my_factor = (a.nsplit == 1 && row_ok) ? lat_row_factor(m, l, tok, h, a.sinks, a.gate, a.ld_gate) : 0.f;
     // the accumulators' rows are 4 g + i: their places and statistics come from the lanes that own those rows
     const long my_out = static_cast<long>(tok) * a.o_ts + static_cast<long>(h) * a.o_hs;
     const long my_pair = static_cast<long>(h) * a.T + tok;           // place in the workspace
@@ -219,9 +245,9 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(LatentArgs a
         const float li = __shfl(l, src, 64), mi = __shfl(m, src, 64);
         const long oo = __shfl(static_cast<int>(my_out), src, 64);   // (pairs * strides stay below 2^31: checked by the entry point)
         const long pp = __shfl(static_cast<int>(my_pair), src, 64);
+        const float inv = __shfl(my_factor, src, 64);
         if (!ok) continue;
         if (a.nsplit == 1) {
-            const float inv = 1.0f / li;
 #pragma unroll
             for (int c = 0; c < RC; ++c)
                 if (c < rc) a.out[oo * a.R + c * 16 + r16] = static_cast<bf16>(acc[c][i] * inv);
@@ -243,7 +269,8 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(LatentArgs a
 // entries of the runs' sums, eight loads asked for at a time.
 __global__ __launch_bounds__(256) void latent_join_kernel(const float* __restrict__ ws_o, const float* __restrict__ ws_ml,
                                                           bf16* __restrict__ out, int T, int n, int R, int nsplit, long o_ts,
-                                                          long o_hs) {
+                                                          long o_hs, const float* __restrict__ sinks,
+                                                          const float* __restrict__ gate, int ld_gate) {
     __shared__ float factor[64];
     const int tok = blockIdx.x, h = blockIdx.y;
     const size_t pairs = static_cast<size_t>(n) * T, pair = static_cast<size_t>(h) * T + tok;
@@ -256,7 +283,7 @@ __global__ __launch_bounds__(256) void latent_join_kernel(const float* __restric
         // (the sum over the runs in the order of the runs: lane 0 adds them up)
         float L = 0.f;
         for (int i = 0; i < nsplit; ++i) L += __shfl(f * lz, i, 64);
-        factor[z] = f / L;
+        factor[z] = f * lat_row_factor(M, L, tok, h, sinks, gate, ld_gate);
     }
     __syncthreads();
     bf16* o = out + (static_cast<long>(tok) * o_ts + static_cast<long>(h) * o_hs) * R;
@@ -342,23 +369,24 @@ extern "C" int llme_latent_attention_mfma(const void* qa, const void* qr, const 
                                           float* ws_ml, const int* positions, const int* q_start, const int* block_table,
                                           int max_blocks, int T, int n_seq, int max_new, int n, int R, int r, int page,
                                           float scale, int window, int nsplit, long q_ts, long q_hs, long o_ts, long o_hs,
-                                          hipStream_t stream) {
+                                          const float* sinks, const float* gate, int ld_gate, hipStream_t stream) {
     if (T <= 0 || n_seq <= 0) return 0;
     const int D = R + r;
     if (n <= 0 || R <= 0 || r < 0 || max_new <= 0 || nsplit <= 0 || nsplit > 64 || n_seq > 65535) return kErrBadArgument;
-    if (R % 16 || D % 32 || r % 8 || page % 16 || D > 576 || R > 512) return kErrUnsupported;
+    if (R % 16 || r % 8 || page % 16 || D > 576 || R > 512) return kErrUnsupported;
+    if (gate != nullptr && ld_gate < n) return kErrBadArgument;
     if (static_cast<long>(T) * n * (R > 2 ? R : 2) >= (1l << 31)) return kErrUnsupported;
     if (nsplit > 1 && (ws_o == nullptr || ws_ml == nullptr)) return kErrBadArgument;
     LatentArgs a{static_cast<const bf16*>(qa), static_cast<const bf16*>(qr), static_cast<const bf16*>(cache),
                  static_cast<bf16*>(out), ws_o, ws_ml, positions, q_start, block_table, max_blocks, T, n, R, r, page, window,
-                 nsplit, q_ts, q_hs, o_ts, o_hs, scale * 1.4426950408889634f};
+                 nsplit, q_ts, q_hs, o_ts, o_hs, scale * kLog2E, sinks, gate, ld_gate};
     int rc;
     if (D <= 128 && R <= 128) rc = launch_latent<4, 8>(a, max_new, n_seq, stream);
     else if (D <= 320 && R <= 256) rc = launch_latent<10, 16>(a, max_new, n_seq, stream);
     else rc = launch_latent<18, 32>(a, max_new, n_seq, stream);
     if (rc != 0 || nsplit == 1) return rc;
     hipLaunchKernelGGL(latent_join_kernel, dim3(T, n), dim3(256), 0, stream, ws_o, ws_ml, static_cast<bf16*>(out), T, n, R, nsplit,
-                       o_ts, o_hs);
+                       o_ts, o_hs, sinks, gate, ld_gate);
     return launch_status();
 }
 

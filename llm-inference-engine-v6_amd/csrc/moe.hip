@@ -1,6 +1,6 @@
 // Mixture of experts: every token runs `top` of E small gated feed-forward layers.
 //
-//   moe_route    logits [T, E] (32-bit) -> per token the `top` experts with the largest scores (softmax over
+//   moe_route    logits [T, E] (32-bit, rows ld apart) -> per token the `top` experts with the largest scores (softmax over
 //                the experts, or a sigmoid of each logit on its own; the lower index wins a tie) and their
 //                weights = score * scale, renormalised over the chosen ones or not; pairs are numbered t * top + k
 //   moe_plan     the pairs grouped by expert: every expert's pairs take a run of places padded to whole
@@ -10,7 +10,8 @@
 //   moe_gemm     per tile of places: rows gathered (token = pair / top, or the place itself) times the
 //                tile's expert's matrix [N, K]; plain or gated (act(gate) * up, gate and up rows in one matrix);
 //                the plain-precision kernel; bfloat16 steps take the grouped instances of the matrix-core tile kernel
-//   moe_combine  out[t] (+)= sum_k weight[t, k] * y[place of (t, k)], k in order (no weights: each counts once)
+//   moe_combine  out[t] (+)= sum_k weight[t, k] * y[place of (t, k)], k in order (no weights: each counts once); where a
+//                shared layer's rows are given, first out[t] (+)= sigmoid(gate[t]) * shared[t]
 //
 // Everything that depends on the routing is read from device memory: a step's launches are the same
 // whatever the tokens choose (grids are sized for the most tiles there can be; workgroups beyond the
@@ -28,13 +29,13 @@ __device__ __forceinline__ float moe_act(float g, int act) {
 
 constexpr int kMoeMaxPerLane = 16;      // experts per lane: up to 1024 experts
 
-__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int T, int E, int top,
+__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int ld, int T, int E, int top,
                                                         float scale, int renorm, int sigmoid, int* __restrict__ ids,
                                                         float* __restrict__ wts) {
     const int lane = threadIdx.x & (kWave - 1);
     const int t = blockIdx.x * 4 + threadIdx.x / kWave;
     if (t >= T) return;
-    const float* z = logits + static_cast<size_t>(t) * E;
+    const float* z = logits + static_cast<size_t>(t) * ld;
     float v[kMoeMaxPerLane];
     float mx = -INFINITY;
 #pragma unroll
@@ -193,12 +194,14 @@ __global__ __launch_bounds__(256) void moe_gemm_kernel(const TA* __restrict__ a,
 
 __global__ void moe_combine_kernel(const float* __restrict__ y, const int* __restrict__ pair_place,
                                    const float* __restrict__ wts, float* __restrict__ out, int top, int H, int accumulate,
+                                   const float* __restrict__ shared, const float* __restrict__ gate, int ld_gate,
                                    size_t total) {
     const size_t idx = static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x;
     if (idx >= total) return;
     const size_t t = idx / H;
     const int c = static_cast<int>(idx % H);
     float s = accumulate ? out[idx] : 0.f;
+    if (shared != nullptr) s += shared[idx] / (1.0f + expf(-gate[t * ld_gate]));
     for (int k = 0; k < top; ++k)
         s = fmaf(wts != nullptr ? wts[t * top + k] : 1.0f, y[static_cast<size_t>(pair_place[t * top + k]) * H + c], s);
     out[idx] = s;
@@ -208,12 +211,12 @@ __global__ void moe_combine_kernel(const float* __restrict__ y, const int* __res
 
 using namespace llme;
 
-extern "C" int llme_moe_route(const float* logits, int T, int E, int top, float scale, int renorm, int sigmoid, int* ids,
+extern "C" int llme_moe_route(const float* logits, int ld, int T, int E, int top, float scale, int renorm, int sigmoid, int* ids,
                               float* wts, hipStream_t stream) {
     if (T <= 0) return 0;
-    if (E <= 0 || top <= 0 || top > E) return kErrBadArgument;
+    if (E <= 0 || top <= 0 || top > E || ld < E) return kErrBadArgument;
     if (E > kMoeMaxPerLane * kWave) return kErrUnsupported;
-    hipLaunchKernelGGL(moe_route_kernel, dim3((T + 3) / 4), dim3(256), 0, stream, logits, T, E, top, scale, renorm, sigmoid, ids, wts);
+    hipLaunchKernelGGL(moe_route_kernel, dim3((T + 3) / 4), dim3(256), 0, stream, logits, ld, T, E, top, scale, renorm, sigmoid, ids, wts);
     return launch_status();
 }
 
@@ -259,11 +262,12 @@ extern "C" int llme_moe_gemm(const void* a, int a_dtype, const void* w, int gate
 }
 
 extern "C" int llme_moe_combine(const float* y, const int* pair_place, const float* wts, float* out, int T, int top,
-                                int H, int accumulate, hipStream_t stream) {
+                                int H, int accumulate, const float* shared, const float* gate, int ld_gate, hipStream_t stream) {
     if (T <= 0) return 0;
+    if (shared != nullptr && (gate == nullptr || ld_gate <= 0)) return kErrBadArgument;
     const size_t total = static_cast<size_t>(T) * H;
     hipLaunchKernelGGL(moe_combine_kernel, dim3(static_cast<unsigned>((total + 255) / 256)), dim3(256), 0, stream, y,
-                       pair_place, wts, out, top, H, accumulate, total);
+                       pair_place, wts, out, top, H, accumulate, shared, gate, ld_gate, total);
     return launch_status();
 }
 

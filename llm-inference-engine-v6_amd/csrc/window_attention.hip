@@ -15,7 +15,8 @@
 // head with a weight over the head's entries where given, or without one (`unit_norm`; a rotation leaves a head's length
 // as it is, so a norm without a weight is the same in front of it and behind it), a rotation of the first `rot` entries by position x
 // frequency, entry i with entry i + rot / 2 or, `pairs` = 1, entry 2 i with entry 2 i + 1; queries times a temperature
-// 1 + coef ln(floor((p + 1) / every) + 1) where `every` > 0; nk = 0: the layer reads another layer's keys and values
+// 1 + coef ln(floor((p + 1) / every) + 1) where `every` > 0; cos and sin times `mag` (1 unless a rotation's frequency
+// scaling asks for more); values that mix with an earlier layer's (`v_mode`); nk = 0: the layer reads another layer's keys and values
 // and only its queries are made), an attention kernel leaves per run of keys the maximum, the sum and the unscaled weighted values of
 // every (token, query head), and `window_attention_finish` joins the runs in a fixed order and applies what a mixer
 // does to a head's result before its output product: nothing, an element-wise sigmoid gate, a sigmoid gate of one
@@ -36,6 +37,18 @@ namespace llme {
 
 constexpr int kMaxHeadEntries = 256;
 
+// Values that mix with those of an earlier layer (value residuals): first [T, nv dv] (32-bit, of this step's tokens) is
+// written by the first such layer (mode 1) and read by the later ones (mode 2): v <- (1 - lam) v + lam first.
+struct ValueMix {
+    float* first;
+    float lam;
+    int mode;
+};
+__device__ __forceinline__ float mixed_value(const ValueMix& mix, float v, size_t at) {
+    if (mix.mode == 1) mix.first[at] = v;
+    return mix.mode == 2 ? fmaf(mix.lam, mix.first[at], (1.0f - mix.lam) * v) : v;
+}
+
 // A workgroup per (token, group of heads): its four wavefronts take the group's heads in turn (queries first, then
 // keys); gridDim.y groups share a token's heads. The angles of the token's position are made once per workgroup.
 // Rows of p: queries at column 0, keys at k_col, values at v_col (v_col < 0: a value head is the key head as
@@ -50,7 +63,7 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict
                                                          const int* __restrict__ positions, const int* __restrict__ seq_idx,
                                                          const int* __restrict__ block_table, int max_blocks,
                                                          TQ* __restrict__ q_out, TC* __restrict__ k_cache, TC* __restrict__ v_cache,
-                                                         int page, int write_v) {
+                                                         int page, int write_v, float mag, ValueMix mix) {
     __shared__ float cs_t[kMaxHeadEntries / 2], sn_t[kMaxHeadEntries / 2];
     const int t = blockIdx.x;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -65,8 +78,8 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict
     for (int f = threadIdx.x; f < half; f += 256) {
         float sn, cs;
         sincosf(fpos * inv_freq[f], &sn, &cs);
-        sn_t[f] = sn;
-        cs_t[f] = cs;
+        sn_t[f] = sn * mag;
+        cs_t[f] = cs * mag;
     }
     __syncthreads();
     // this lane's entries: whether they turn, with which partner, which way, the norms' weights
@@ -139,7 +152,8 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(const float* __restrict
     if (write_v && v_col >= 0 && nv > 0) {
         const float* vp = row + v_col;
         for (int e = blockIdx.y * 256 + threadIdx.x; e < nv * dv; e += 256 * gridDim.y)
-            v_cache[((static_cast<size_t>(pg) * nv + e / dv) * dv + e % dv) * page + in_page] = from_float<TC>(vp[e]);
+            v_cache[((static_cast<size_t>(pg) * nv + e / dv) * dv + e % dv) * page + in_page] =
+                from_float<TC>(mixed_value(mix, vp[e], static_cast<size_t>(t) * nv * dv + e));
     }
 }
 
@@ -150,7 +164,7 @@ template <typename TC>
 __global__ __launch_bounds__(256) void v_write_kernel(const float* __restrict__ p, int ld, int v_col, int nv, int dv,
                                                       const int* __restrict__ positions, const int* __restrict__ q_start,
                                                       const int* __restrict__ block_table, int max_blocks, TC* __restrict__ v_cache,
-                                                      int page) {
+                                                      int page, ValueMix mix) {
     const int s = blockIdx.y;
     const int e = blockIdx.z * 256 + threadIdx.x;
     const int row0 = q_start[s], n = q_start[s + 1] - row0;
@@ -166,7 +180,10 @@ __global__ __launch_bounds__(256) void v_write_kernel(const float* __restrict__ 
     Piece piece;
 #pragma unroll
     for (int j = 0; j < 8; ++j)
-        if (j >= lo && j < hi) piece.x[j] = from_float<TC>(src[static_cast<size_t>(row0 + base + j - ctx) * ld]);
+        if (j >= lo && j < hi) {
+            const size_t t = static_cast<size_t>(row0 + base + j - ctx);
+            piece.x[j] = from_float<TC>(mixed_value(mix, src[t * ld], t * nv * dv + e));
+        }
     if (lo == 0 && hi == 8) {
         *reinterpret_cast<Piece*>(dst) = piece;
     } else {
@@ -410,8 +427,10 @@ extern "C" int llme_qk_prepare(const float* p, int ld, int nq, int nk, int nv, i
                                const void* wq, const void* wk, int w_dtype, int unit_norm, float eps, const float* inv_freq, int rot,
                                int pairs, float qt_coef, int qt_every, const int* positions, const int* seq_idx, const int* block_table, int max_blocks, void* q_out,
                                int q_dtype, void* k_cache, void* v_cache, int cache_dtype, int page, int T, const int* q_start,
-                               int n_seq, int max_new, hipStream_t stream) {
+                               int n_seq, int max_new, float mag, float* v_first, float v_lam, int v_mode, hipStream_t stream) {
     if (T <= 0) return 0;
+    if (v_mode < 0 || v_mode > 2 || (v_mode && (v_first == nullptr || v_col < 0 || nv <= 0))) return kErrBadArgument;
+    const ValueMix mix{v_first, v_lam, v_mode};
     if (dk <= 0 || page <= 0 || rot < 0 || rot > dk || rot % 2 != 0 || qt_every < 0) return kErrBadArgument;
     if (nk > 0 && (dv <= 0 || nv <= 0 || nk % nv != 0 || k_cache == nullptr || v_cache == nullptr)) return kErrBadArgument;
     if (nk == 0) nv = 0;                    // (queries only: the keys and values are another layer's)
@@ -435,7 +454,7 @@ extern "C" int llme_qk_prepare(const float* p, int ld, int nq, int nk, int nv, i
 #define LLME_PREP_E(TQ, TC, TW, EPL)                                                                                              \
     hipLaunchKernelGGL((qk_prepare_kernel<TQ, TC, TW, EPL>), grid, dim3(256), 0, stream, p, ld, nq, nk, nv, dk, dv, k_col, v_col, \
                        static_cast<const TW*>(wq), static_cast<const TW*>(wk), unit_norm, eps, inv_freq, rot, pairs, qt_coef, qt_every, positions, seq_idx, \
-                       block_table, max_blocks, static_cast<TQ*>(q_out), static_cast<TC*>(k_cache), static_cast<TC*>(v_cache), page, octets == 0)
+                       block_table, max_blocks, static_cast<TQ*>(q_out), static_cast<TC*>(k_cache), static_cast<TC*>(v_cache), page, octets == 0, mag, mix)
     if (q_dtype != cache_dtype) return kErrBadArgument;
     if (q_dtype == kF32 && w_dtype == kF32) LLME_PREP(float, float, float);
     else if (q_dtype == kBF16 && w_dtype == kF32) LLME_PREP(bf16, bf16, float);
@@ -447,10 +466,10 @@ extern "C" int llme_qk_prepare(const float* p, int ld, int nq, int nk, int nv, i
         const dim3 vgrid(octets, n_seq, (nv * dv + 255) / 256);
         if (cache_dtype == kF32)
             hipLaunchKernelGGL((v_write_kernel<float>), vgrid, dim3(256), 0, stream, p, ld, v_col, nv, dv, positions, q_start, block_table,
-                               max_blocks, static_cast<float*>(v_cache), page);
+                               max_blocks, static_cast<float*>(v_cache), page, mix);
         else
             hipLaunchKernelGGL((v_write_kernel<bf16>), vgrid, dim3(256), 0, stream, p, ld, v_col, nv, dv, positions, q_start, block_table,
-                               max_blocks, static_cast<bf16*>(v_cache), page);
+                               max_blocks, static_cast<bf16*>(v_cache), page, mix);
     }
     return launch_status();
 }

@@ -5,5 +5,6 @@ from . import bidirax  # registers "Bidirax"
 from . import zetonex  # registers "Zetonex"
 from . import zapolorn  # registers "Zapolorn"
 from . import lukupel  # registers "Lukupel"
+from . import diporax  # registers "Diporax"
 
-__all__ = ["DecoderModel", "LayerCall", "llama", "rilonex", "bidirax", "zetonex", "zapolorn", "lukupel"]
+__all__ = ["DecoderModel", "LayerCall", "llama", "rilonex", "bidirax", "zetonex", "zapolorn", "lukupel", "diporax"]

@@ -34,7 +34,7 @@ class DecoderModel(Part):
 
     def __init__(self, config, embedding: TokenEmbedding, layers: list[Block], final_norm: Norm,
                  head: Head, schedule: list[LayerCall] | None = None, names: dict | None = None, streams: int = 0,
-                 pass_input: Part | None = None, layer_numbers: list[int] | None = None):
+                 pass_input: Part | None = None, layer_numbers: list[int] | None = None, shared: dict[str, Part] | None = None):
         self.config = config
         # streams > 0: the residual is kept as that many streams [streams, T, H] (blocks that know how read and
         # write them); every stream starts as the embedding, and the final norm reads their sum
@@ -49,6 +49,8 @@ class DecoderModel(Part):
         # what runs in front of the calls marked `enter`: forward(h, h0, step) replaces the stream h, given the
         # embedding's output h0 (a stack of layers that runs several passes over the same weights)
         self.pass_input = pass_input
+        # parts with tensors that several layers read (name prefix -> part): they run where the layers use them
+        self.shared = dict(shared or {})
         if any(call.enter for call in self.schedule) and (pass_input is None or self.streams):
             raise ValueError("a schedule with passes needs the model's pass-input map (and a single stream)")
         for call in self.schedule:
@@ -70,6 +72,7 @@ class DecoderModel(Part):
         out[n["head"]] = self.head
         if self.pass_input is not None:
             out[n["pass_input"]] = self.pass_input
+        out.update(self.shared)
         return out
 
     def aliases(self):

@@ -21,11 +21,11 @@ declare("llme_scale_f32", [_vp, _z, _f, _vp])
 declare("llme_latent_prepare", [_vp, _i, _i, _i, _i, _i, _vp, _vp, _i, _vp, _f, _vp, _vp, _vp, _i, _vp, _vp, _i, _i, _i, _f, _vp])
 declare("llme_latent_q_rotate", [_vp, _i, _vp, _f, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp])
 declare("llme_head_gemm", [_vp, _i, _l, _l, _vp, _i, _vp, _i, _l, _l, _i, _i, _i, _i, _vp])
-declare("llme_latent_attention", [_vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _f, _i, _vp])
-declare("llme_moe_route", [_vp, _i, _i, _i, _f, _i, _i, _vp, _vp, _vp])
+declare("llme_latent_attention", [_vp, _i, _vp, _i, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _f, _i, _vp, _vp, _i, _vp])
+declare("llme_moe_route", [_vp, _i, _i, _i, _i, _f, _i, _i, _vp, _vp, _vp])
 declare("llme_moe_plan", [_vp, _i, _i, _i, _i, _vp, _vp, _vp, _vp, _vp])
 declare("llme_moe_gemm", [_vp, _i, _vp, _i, _i, _vp, _i, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _vp])
-declare("llme_moe_combine", [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp])
+declare("llme_moe_combine", [_vp, _vp, _vp, _vp, _i, _i, _i, _i, _vp, _vp, _i, _vp])
 
 
 # --- sandwich norm ---------------------------------------------------------------------
@@ -135,13 +135,22 @@ def latent_attention_fits(kv_rank: int, rot: int) -> bool:
     return kv_rank <= LATENT_MAX_RANK and kv_rank + rot <= LATENT_MAX_ROW
 
 
-_fast_latent_attention = None   # set by ops/latent_mfma.py
+def _sinks_and_gate(sinks: torch.Tensor | None, gate: torch.Tensor | None, T: int, heads: int) -> int:
+    """Checks them; returns the gate's row stride."""
+    if sinks is not None:
+        require(sinks, "sinks", torch.float32, (heads,))
+    if gate is None:
+        return 0
+    from .recurrent import _cols
+    return _cols(gate, "gate", torch.float32, T, heads)
 
 
 def latent_attention(qp: torch.Tensor, cache: torch.Tensor, out: torch.Tensor, step, block_table: torch.Tensor,
-                     heads: int, kv_rank: int, scale: float, window: int = 0) -> None:
+                     heads: int, kv_rank: int, scale: float, window: int = 0, sinks: torch.Tensor | None = None,
+                     gate: torch.Tensor | None = None) -> None:
     """out[t, h] = sum_j softmax_j(scale qp[t, h] . row_j) row_j[:kv_rank] over the rows of the token's request
-    that it may see (all up to its own; with a window the last `window` of them)."""
+    that it may see (all up to its own; with a window the last `window` of them). sinks [heads] (32-bit): the softmax's
+    sum also holds e^(sink); gate [T, heads] (32-bit, a column range): times sigmoid(gate)."""
     T = qp.shape[0]
     require(cache, "cache", _FLOATS, (None, None, None))
     D = cache.shape[2]
@@ -150,29 +159,28 @@ def latent_attention(qp: torch.Tensor, cache: torch.Tensor, out: torch.Tensor, s
     require(block_table, "block_table", torch.int32, (None, None))
     if not latent_attention_fits(kv_rank, D - kv_rank):
         raise KernelError(f"latent attention: rows of {D} with a latent of {kv_rank} are beyond the kernel's limits")
-    if _fast_latent_attention is not None and _fast_latent_attention(qp, cache, out, step, block_table, heads, kv_rank,
-                                                                     scale, window):
-        return
+    ld_gate = _sinks_and_gate(sinks, gate, T, heads)
     check(entry("llme_latent_attention")(ptr(qp), code(qp.dtype), ptr(cache), code(cache.dtype), ptr(out),
                                          ptr(step.positions), ptr(step.seq_idx), ptr(block_table), block_table.shape[1],
-                                         T, heads, kv_rank, D, cache.shape[1], float(scale), int(window), stream()),
+                                         T, heads, kv_rank, D, cache.shape[1], float(scale), int(window), ptr(sinks), ptr(gate), ld_gate,
+                                         stream()),
           "latent_attention")
 
 
 # --- latent attention on the matrix cores ------------------------------------------------
 declare("llme_latent_attention_mfma", [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i,
-                                       _l, _l, _l, _l, _vp])
+                                       _l, _l, _l, _l, _vp, _vp, _i, _vp])
 declare("llme_latent_q_split", [_vp, _vp, _f, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp])
 declare("llme_heads_to_rows", [_vp, _vp, _i, _i, _i, _vp])
 LATENT_MFMA_MAX_ROW, LATENT_MFMA_MAX_RANK = 576, 512
 
 
 def latent_mfma_fits(cache: torch.Tensor, kv_rank: int, rot: int, choices=None) -> bool:
-    """Whether the matrix-core kernel takes these rows: bfloat16, a latent that is a multiple of 16, rows a multiple of 32,
-    pages a multiple of 16."""
+    """Whether the matrix-core kernel takes these rows: bfloat16, a latent that is a multiple of 16, a rotated part that is
+    one of 8, pages a multiple of 16."""
     from .choices import DEFAULT
     D = kv_rank + rot
-    return ((choices or DEFAULT).fast_attention and cache.dtype == torch.bfloat16 and kv_rank % 16 == 0 and D % 32 == 0 and rot % 8 == 0
+    return ((choices or DEFAULT).fast_attention and cache.dtype == torch.bfloat16 and kv_rank % 16 == 0 and rot % 8 == 0
             and cache.shape[1] % 16 == 0 and D <= LATENT_MFMA_MAX_ROW and kv_rank <= LATENT_MFMA_MAX_RANK)
 
 
@@ -194,8 +202,10 @@ def latent_splits(step, heads: int, window: int) -> tuple[int, int]:
 
 
 def latent_attention_mfma(qa: torch.Tensor, qr: torch.Tensor | None, cache: torch.Tensor, out: torch.Tensor, step,
-                          block_table: torch.Tensor, heads: int, kv_rank: int, scale: float, window: int, head_major: bool) -> None:
-    """The matrix-core kernel. qa [T, heads, kv_rank] and qr [T, heads, rot] (head_major: [heads, T, ..]); out as qa."""
+                          block_table: torch.Tensor, heads: int, kv_rank: int, scale: float, window: int, head_major: bool,
+                          sinks: torch.Tensor | None = None, gate: torch.Tensor | None = None) -> None:
+    """The matrix-core kernel. qa [T, heads, kv_rank] and qr [T, heads, rot] (head_major: [heads, T, ..]); out as qa; sinks and
+    gate as in `latent_attention`."""
     T = step.num_tokens
     D = cache.shape[2]
     rot = D - kv_rank
@@ -206,6 +216,7 @@ def latent_attention_mfma(qa: torch.Tensor, qr: torch.Tensor | None, cache: torc
         raise KernelError("latent attention: the queries do not fit the step")
     if rot:
         require(qr, "qr", torch.bfloat16)
+    ld_gate = _sinks_and_gate(sinks, gate, T, heads)
     max_new, nsplit = latent_splits(step, heads, window)
     ws_o = ws_ml = None
     if nsplit > 1:
@@ -215,7 +226,7 @@ def latent_attention_mfma(qa: torch.Tensor, qr: torch.Tensor | None, cache: torc
     check(entry("llme_latent_attention_mfma")(
         ptr(qa), ptr(qr) if rot else None, ptr(cache), ptr(out), ptr(ws_o), ptr(ws_ml), ptr(step.positions), ptr(step.q_start),
         ptr(block_table), block_table.shape[1], T, step.num_seqs, max_new, heads, kv_rank, rot, cache.shape[1], float(scale),
-        int(window), nsplit, ts, hs, ts, hs, stream()), "latent_attention_mfma")
+        int(window), nsplit, ts, hs, ts, hs, ptr(sinks), ptr(gate), ld_gate, stream()), "latent_attention_mfma")
 
 
 def latent_q_split(q: torch.Tensor, freq: torch.Tensor | None, mag: float, positions: torch.Tensor, qn: torch.Tensor,
@@ -284,15 +295,16 @@ def moe_capacity(pairs: int, experts: int, tile: int = MOE_TILE) -> int:
 
 def moe_route(logits: torch.Tensor, top: int, scale: float, renormalize: bool, ids: torch.Tensor, wts: torch.Tensor,
               scoring: str = "softmax") -> None:
-    """ids, wts [T, top]: every row's `top` experts with the largest scores, softmax over the row or ("sigmoid") a
+    """logits [T, E] 32-bit (a column range of a wider buffer); ids, wts [T, top]: every row's `top` experts with the largest scores, softmax over the row or ("sigmoid") a
     sigmoid of each logit, and their weights score * scale (over the chosen scores' sum first where `renormalize`)."""
     if scoring not in ("softmax", "sigmoid"):
         raise KernelError(f"moe_route: scoring {scoring!r} is neither 'softmax' nor 'sigmoid'")
-    require(logits, "logits", torch.float32, (None, None))
+    from .recurrent import _cols
     T, E = logits.shape
+    ld = _cols(logits, "logits", torch.float32)
     require(ids, "ids", torch.int32, (T, top))
     require(wts, "wts", torch.float32, (T, top))
-    check(entry("llme_moe_route")(ptr(logits), T, E, top, float(scale), 1 if renormalize else 0, 1 if scoring == "sigmoid" else 0,
+    check(entry("llme_moe_route")(ptr(logits), ld, T, E, top, float(scale), 1 if renormalize else 0, 1 if scoring == "sigmoid" else 0,
                                   ptr(ids), ptr(wts), stream()),
           "moe_route")
 
@@ -365,8 +377,9 @@ def moe_gemm_clamped(a: torch.Tensor, w: torch.Tensor, group: int, out: torch.Te
 
 
 def moe_combine(y: torch.Tensor, pair_place: torch.Tensor, wts: torch.Tensor | None, out: torch.Tensor, accumulate: bool,
-                top: int | None = None) -> None:
-    """out[t] (+)= sum_k wts[t, k] y[place of pair (t, k)]; wts None: every one of a token's `top` results counts once."""
+                top: int | None = None, shared: torch.Tensor | None = None, shared_gate: torch.Tensor | None = None) -> None:
+    """out[t] (+)= sum_k wts[t, k] y[place of pair (t, k)]; wts None: every one of a token's `top` results counts once.
+    shared [T, H] with shared_gate [T, 1] (both 32-bit, the gate a column of a wider buffer): also sigmoid(gate) * shared."""
     require(out, "out", torch.float32, (None, None))
     T, H = out.shape
     if wts is not None:
@@ -376,5 +389,13 @@ def moe_combine(y: torch.Tensor, pair_place: torch.Tensor, wts: torch.Tensor | N
         raise KernelError("moe_combine: without weights the number of results a token has must be given")
     require(y, "y", torch.float32, (None, H))
     require(pair_place, "pair_place", torch.int32, (T * top,))
-    check(entry("llme_moe_combine")(ptr(y), ptr(pair_place), ptr(wts), ptr(out), T, top, H, 1 if accumulate else 0, stream()),
+    if (shared is None) != (shared_gate is None):
+        raise KernelError("moe_combine: a shared layer's rows and their gate come together")
+    ld_gate = 0
+    if shared is not None:
+        from .recurrent import _cols
+        require(shared, "shared", torch.float32, (T, H))
+        ld_gate = _cols(shared_gate, "shared_gate", torch.float32, T, 1)
+    check(entry("llme_moe_combine")(ptr(y), ptr(pair_place), ptr(wts), ptr(out), T, top, H, 1 if accumulate else 0, ptr(shared),
+                                    ptr(shared_gate), ld_gate, stream()),
           "moe_combine")

@@ -17,7 +17,7 @@ FINISH_MODES = {"plain": 0, "gate": 1, "difference": 2, "head_gate": 3}
 BIAS_ACTIVATIONS = {"silu": 0, "relu": 1, "gelu_tanh": 2, "swish_clamped": 3}
 
 declare("llme_qk_prepare", [_vp, _i, _i, _i, _i, _i, _i, _i, _i, _vp, _vp, _i, _i, _f, _vp, _i, _i, _f, _i, _vp, _vp, _vp, _i, _vp, _i, _vp,
-                            _vp, _i, _i, _i, _vp, _i, _i, _vp])
+                            _vp, _i, _i, _i, _vp, _i, _i, _f, _vp, _f, _i, _vp])
 declare("llme_window_attention", [_vp, _i, _vp, _vp, _i, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i, _i, _vp,
                                   _vp])
 declare("llme_window_attention_finish", [_vp, _vp, _i, _i, _i, _i, _i, _i, _vp, _i, _f, _f, _f, _vp, _vp, _i, _i, _vp])
@@ -37,13 +37,15 @@ def _columns(p: torch.Tensor, name: str) -> int:
 def qk_prepare(p: torch.Tensor, step, block_table: torch.Tensor | None, q_out: torch.Tensor, k_cache: torch.Tensor | None,
                v_cache: torch.Tensor | None, nq: int, k_col: int, v_col: int | None, inv_freq: torch.Tensor | None, rot: int,
                wq: torch.Tensor | None = None, wk: torch.Tensor | None = None, eps: float = 0.0, pairs: str = "halves",
-               q_temp: tuple[float, int] | None = None, dk: int | None = None, unit_norm: bool = False) -> None:
+               q_temp: tuple[float, int] | None = None, dk: int | None = None, unit_norm: bool = False, mag: float = 1.0,
+               v_first: torch.Tensor | None = None, v_mix: float | None = None) -> None:
     """Rows p [T, ..] (32-bit: nq query heads of dk entries at column 0, the key heads at k_col, the value heads at
     v_col; v_col None: a value head is the key head as projected) -> q_out [T, nq dk] and the cache entries of the
     rows' tokens: k_cache [pages, nk, page, dk], v_cache [pages, nv, dv, page]. wq, wk [dk]: every query and key
     head is divided by its root mean square (eps inside the root) and multiplied by the weight first; unit_norm: the same without a weight. Then the first
     `rot` entries of a query or key head turn by position * inv_freq[i]: entry i with entry i + rot / 2 (pairs
-    "halves") or entry 2 i with entry 2 i + 1 ("neighbours"). q_temp (coef, every): the queries of position p times
+    "halves") or entry 2 i with entry 2 i + 1 ("neighbours"), cos and sin times mag. v_first [T, nv dv] (32-bit) with v_mix
+    None: the values are also left there; with a number: they become (1 - v_mix) v + v_mix v_first. q_temp (coef, every): the queries of position p times
     1 + coef ln(floor((p + 1) / every) + 1). k_cache None: only the queries are made (the keys and values are another
     layer's; `dk` then says the heads' size)."""
     T = p.shape[0]
@@ -77,6 +79,14 @@ def qk_prepare(p: torch.Tensor, step, block_table: torch.Tensor | None, q_out: t
         require(wq, "wq", _FLOATS, (dk,))
     if wk is not None:
         require(wk, "wk", wq.dtype, (dk,))
+    v_mode = 0
+    if v_first is not None:
+        if k_cache is None or v_col is None:
+            raise KernelError("qk_prepare: values that mix with another layer's are projected values of the layer's own")
+        require(v_first, "v_first", torch.float32, (T, nv * dv))
+        v_mode = 1 if v_mix is None else 2
+    elif v_mix is not None:
+        raise KernelError("qk_prepare: v_mix needs the values to mix with")
     coef, every = (float(q_temp[0]), int(q_temp[1])) if q_temp else (0.0, 0)
     if q_temp and every <= 0:
         raise KernelError("qk_prepare: the queries' temperature steps every > 0 positions")
@@ -85,7 +95,8 @@ def qk_prepare(p: torch.Tensor, step, block_table: torch.Tensor | None, q_out: t
                                    1 if pairs == "neighbours" else 0, coef, every,
                                    ptr(step.positions), ptr(step.seq_idx), ptr(block_table) if nk else None,
                                    block_table.shape[1] if nk else 0, ptr(q_out), code(q_out.dtype), ptr(k_cache), ptr(v_cache),
-                                   code(q_out.dtype), page, T, ptr(step.q_start), step.num_seqs, max(step.new_lens), stream()), "qk_prepare")
+                                   code(q_out.dtype), page, T, ptr(step.q_start), step.num_seqs, max(step.new_lens), float(mag), ptr(v_first), 0.0 if v_mix is None else float(v_mix),
+                                   v_mode, stream()), "qk_prepare")
 
 
 declare("llme_window_attention_mfma", [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _i, _i,

@@ -6,6 +6,7 @@ from .rope import RotaryEmbedding, inverse_frequencies
 from .embedding import Embedding, OutputHead
 from .mlp import GatedMLP, SquaredReluMLP
 from .attention import Attention
+from .token_input import TokenInput, TokenTable
 from .block import OutputNormBlock, ParallelBlock, PreNormBlock, SandwichBlock
 from .projected import ParallelMixer, ProjectedMixer
 from .rglru import RGLRU
@@ -15,7 +16,7 @@ from .hyper import HyperConnectionBlock
 from .latent_attention import LatentAttention
 from .moe import MixtureOfExperts
 from .window_attention import WindowAttention
-from .linear_attention import GatedLinearAttention
+from .linear_attention import GatedLinearAttention, LightningAttention
 from .mlstm import MatrixMemory
 from .reentry import PassInput
 
@@ -24,4 +25,5 @@ __all__ = ["PAGE", "Block", "CacheSpec", "FeedForward", "LayerCache", "Mixer", "
            "register_part", "registered", "RMSNorm", "RotaryEmbedding", "inverse_frequencies", "Embedding",
            "OutputHead", "GatedMLP", "Attention", "PreNormBlock", "ParallelMixer", "ProjectedMixer", "RGLRU", "GatedDeltaRule",
            "SigmoidAttention", "HyperConnectionBlock", "CenteredRMSNorm", "SandwichBlock", "LatentAttention",
-           "MixtureOfExperts", "WindowAttention", "PassInput", "ParallelBlock", "OutputNormBlock", "GatedLinearAttention", "MatrixMemory", "SquaredReluMLP"]
+           "MixtureOfExperts", "WindowAttention", "PassInput", "ParallelBlock", "OutputNormBlock", "GatedLinearAttention", "LightningAttention", "MatrixMemory",
+           "SquaredReluMLP", "TokenInput", "TokenTable"]

@@ -9,8 +9,9 @@ from __future__ import annotations
 import torch
 
 from .. import ops
-from .base import Block, FeedForward, Mixer, Norm
+from .base import Block, FeedForward, Mixer, Norm, ParamSpec
 from .registry import register_part
+from .token_input import TokenInput
 
 
 class PreNormBlock(Block):
@@ -141,7 +142,9 @@ class ParallelBlock(Block):
 
 class OutputNormBlock(Block):
     """Norms behind the sublayers only: h += c norm1(mixer(h)); h += c norm2(ffn(h)) with a constant c (`residual_scale`, 1
-    unless given). The sublayers read the stream itself
+    unless given). `layer_scale`: what a sublayer adds is multiplied entry by entry by a vector of its own ("ls1", "ls2"; made
+    part of the norm's weight, a 32-bit product, when the tensors are loaded). `token_input`: a third sublayer behind the
+    other two, the layer's own input from the token's id, normed and added the same way without scale or vector. The sublayers read the stream itself
     (rounded to the activation type where that is not 32-bit); a sublayer's result is a 32-bit buffer of its own, and
     the norm behind it, the sum into the stream and the copy of the updated rows that the next sublayer reads (this
     block's feed-forward, or the mixer of the block behind) are one kernel."""
@@ -149,11 +152,15 @@ class OutputNormBlock(Block):
     ADDED_ROWS = 64             # steps of up to this many rows add the parts of a sublayer's last product
 
     def __init__(self, mixer: Mixer, feed_forward: FeedForward | None, mixer_norm: Norm, ffn_norm: Norm | None,
-                 names: dict | None = None, residual_scale: float = 1.0):
+                 names: dict | None = None, residual_scale: float = 1.0, layer_scale: bool = False,
+                 token_input: TokenInput | None = None):
         self.mixer, self.feed_forward = mixer, feed_forward
         self.mixer_norm, self.ffn_norm = mixer_norm, ffn_norm
         self.residual_scale = float(residual_scale)
-        self.names = {"mixer_norm": "norm1", "mixer": "mix", "ffn_norm": "norm2", "feed_forward": "mlp"}
+        self.layer_scale, self.token_input = bool(layer_scale), token_input
+        self.scales: list[torch.Tensor] = []
+        self.names = {"mixer_norm": "norm1", "mixer": "mix", "ffn_norm": "norm2", "feed_forward": "mlp", "mixer_scale": "ls1",
+                      "ffn_scale": "ls2", "token_input": "side"}
         if names:
             self.names.update(names)
         # the block that runs behind this one (told by the model as it runs its schedule; None: unknown)
@@ -164,14 +171,33 @@ class OutputNormBlock(Block):
         out = {n["mixer_norm"]: self.mixer_norm, n["mixer"]: self.mixer}
         if self.feed_forward is not None:
             out.update({n["ffn_norm"]: self.ffn_norm, n["feed_forward"]: self.feed_forward})
+        if self.token_input is not None:
+            out[n["token_input"]] = self.token_input
         return out
 
-    def _join(self, y, post: Norm, h, x, clear: bool) -> None:
-        """h += c post(y), and x = the updated rows where x is another buffer than the stream."""
+    def _scaled_norms(self) -> list[tuple[str, Norm]]:
+        n = self.names
+        out = [(n["mixer_scale"], self.mixer_norm)]
+        return out + [(n["ffn_scale"], self.ffn_norm)] if self.feed_forward is not None else out
+
+    def param_specs(self):
+        if not self.layer_scale:
+            return {}
+        return {name: ParamSpec((norm.size,), "norm") for name, norm in self._scaled_norms()}
+
+    def load_tree(self, get, placement, prefix=""):
+        super().load_tree(get, placement, prefix)
+        if self.layer_scale:
+            f32 = torch.float32
+            self.scales = [placement.place(get(prefix + name), f32) * norm.fused_rms()[0].to(f32) for name, norm in self._scaled_norms()]
+
+    def _join(self, y, post: Norm, h, x, clear: bool, c: float = 1.0, weight: torch.Tensor | None = None) -> None:
+        """h += c post(y), and x = the updated rows where x is another buffer than the stream; weight: in place of the norm's
+        (its product with the sublayer's vector)."""
         rms = post.fused_rms()
         if rms is None:
             raise NotImplementedError("output-norm blocks take norms of the plain RMS formula behind their sublayers")
-        ops.norm_add(y, rms[0], h, rms[1], None, x if x is not h else None, self.residual_scale, clear)
+        ops.norm_add(y, rms[0] if weight is None else weight, h, rms[1], None, x if x is not h else None, c, clear)
 
     def forward(self, h, step, cache, write_cache=True):
         T, H = h.shape
@@ -193,12 +219,16 @@ class OutputNormBlock(Block):
                 ops.copy_cols(h, x)
         self.mixer.forward(x, step, cache, y, add, write_cache)
         hand_on = isinstance(self.next_block, OutputNormBlock) and x is not h
-        if self.feed_forward is None:
-            self._join(y, self.mixer_norm, h, x if hand_on else h, add)
-        else:
-            self._join(y, self.mixer_norm, h, x, add)
+        c, scales = self.residual_scale, self.scales or [None, None]
+        # (the last sum into the stream leaves the copy of the rows only where the block behind reads it)
+        last = 2 if self.token_input is not None else 1 if self.feed_forward is not None else 0
+        self._join(y, self.mixer_norm, h, x if hand_on or last > 0 else h, add, c, scales[0])
+        if self.feed_forward is not None:
             self.feed_forward.forward(x, step, y, add)
-            self._join(y, self.ffn_norm, h, x if hand_on else h, add)
+            self._join(y, self.ffn_norm, h, x if hand_on or last > 1 else h, add, c, scales[1])
+        if self.token_input is not None:
+            self.token_input.forward(x, step, y, add)
+            self._join(y, self.token_input.norm, h, x if hand_on else h, add)
         if hand_on:
             step.extra["block.stream_copy is for"] = id(self.next_block)
 

@@ -9,30 +9,41 @@ from __future__ import annotations
 import torch
 
 from .. import ops
-from .base import Getter, Head, ParamSpec, Placement, TokenEmbedding
+from .base import Getter, Head, Norm, ParamSpec, Placement, TokenEmbedding
 from .registry import register_part
 
 
 class Embedding(TokenEmbedding):
     graph_safe = True
 
-    def __init__(self, vocab_size: int, hidden_size: int, tensor: str = "weight", scale: float = 1.0):
+    def __init__(self, vocab_size: int, hidden_size: int, tensor: str = "weight", scale: float = 1.0, norm: Norm | None = None):
         self.vocab_size, self.hidden_size = int(vocab_size), int(hidden_size)
         self.tensor = tensor            # the local name of the table ("": the part's own name)
+        self.norm = norm                # what the (scaled) rows pass before they become the stream ("norm")
         self.scale = float(scale)       # a multiplier on every row, applied in 32-bit
         self.weight: torch.Tensor | None = None
 
     def param_specs(self):
         return {self.tensor: ParamSpec((self.vocab_size, self.hidden_size), "linear")}
 
+    def children(self):
+        return {"norm": self.norm} if self.norm is not None else {}
+
     def load_params(self, get: Getter, placement: Placement) -> None:
         # (a tied head reads the table as a weight matrix: the gather takes either layout)
         self.weight = placement.place_matrix(get(self.tensor))
 
     def forward(self, tokens: torch.Tensor, out: torch.Tensor, step=None) -> None:
-        ops.embed_gather(self.weight, tokens, out)
+        rms = self.norm.fused_rms() if self.norm is not None else None
+        if rms is not None and self.scale == 1.0 and self.hidden_size <= ops.token_input.EMBED_NORM_MAX_WIDTH:
+            ops.token_input.embed_norm(self.weight, tokens, rms[0], rms[1], out)
+            return
+        rows = out if self.norm is None else step.buffer("embedding.rows", tuple(out.shape), torch.float32)
+        ops.embed_gather(self.weight, tokens, rows)
         if self.scale != 1.0:
-            ops.scale_(out, self.scale)
+            ops.scale_(rows, self.scale)
+        if self.norm is not None:
+            self.norm.forward(rows, out)
 
 
 class OutputHead(Head):

@@ -5,7 +5,10 @@ the heads' queries, each [dim unrotated | rot_dim rotated] entries. It also goes
 entries: the first kv_rank, RMS-normed, are the latent c; the last rot_dim, rotated at the token's position,
 are a key part that every head shares. Head h's key is [Wuk_h c | shared part], its value Wuv_h c; scores are
 scale * q . k over the keys the token may see (all earlier ones, or the last `window`), weights their softmax;
-the heads' results side by side go through the output matrix.
+the heads' results side by side go through the output matrix. `sink`: a learned number per head ("sink") whose
+exponential joins the softmax's denominator, a key that is not scaled and has no value. `gate="heads"`: head h's result
+is multiplied by sigmoid(Wg x)_h ("g", one row a head), in front of the output matrix (the attention kernels multiply the
+weighted sum by it, which the value map passes on).
 
 Only c and the shared part are cached: a page holds rows of kv_rank + rot_dim entries. The kernels never
 expand a key or a value either: a query takes Wuk_h^T onto itself and is scored against the rows as they
@@ -21,31 +24,13 @@ and sin times 0.1 ln(factor) + 1. Angles are 32-bit products in the kernels; the
 """
 from __future__ import annotations
 
-import math
-
 import torch
 
 from .. import ops
 from .base import PAGE, CacheSpec, Getter, Mixer, ParamSpec, Placement
+from .frequencies import ramped_frequencies
 from .projected import stack_rows
 from .registry import register_part
-
-
-def ramped_frequencies(dims: int, base: float, scaling: dict | None) -> tuple[torch.Tensor, float]:
-    """([dims / 2] float64 angular steps, the factor on cos and sin)."""
-    i = torch.arange(dims // 2, dtype=torch.float64)
-    f = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / dims)
-    if not scaling:
-        return f, 1.0
-    factor, original = float(scaling["factor"]), float(scaling["original"])
-
-    def pair_of(turns: float) -> float:
-        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
-
-    lo = max(math.floor(pair_of(float(scaling["fast"]))), 0)
-    hi = min(math.ceil(pair_of(float(scaling["slow"]))), dims - 1)
-    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp_(0.0, 1.0)
-    return f / factor * ramp + f * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
 
 
 class LatentAttention(Mixer):
@@ -53,7 +38,11 @@ class LatentAttention(Mixer):
 
     def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int, kv_rank: int, q_rank: int, scale: float,
                  eps: float, rot_dim: int = 0, rot: dict | None = None, window: int = 0, keeps_latent: bool = True,
-                 cache_window: int | None = None):
+                 cache_window: int | None = None, sink: bool = False, gate: bool | str = False):
+        if gate not in (False, "heads"):
+            raise ValueError(f"gate {gate!r} is neither False nor 'heads'")
+        self.sink, self.gate = bool(sink), gate
+        self.sinks: torch.Tensor | None = None
         if rot_dim % 2:
             raise ValueError(f"rot_dim {rot_dim} must be even")
         if rot_dim and not rot:
@@ -84,6 +73,10 @@ class LatentAttention(Mixer):
                "o": ParamSpec((H, n * self.vdim))}
         if self.keeps_latent:
             out.update({"dkv": ParamSpec((self.row, H)), "dkv.norm": ParamSpec((self.kv_rank,), "norm")})
+        if self.sink:
+            out["sink"] = ParamSpec((n,))
+        if self.gate:
+            out["g"] = ParamSpec((n, H))
         return out
 
     def refusals(self):
@@ -100,7 +93,9 @@ class LatentAttention(Mixer):
 
     def load_params(self, get: Getter, placement: Placement) -> None:
         n, d, dv, R = self.heads, self.dim, self.vdim, self.kv_rank
-        downs = [get("dq")] + ([get("dkv")] if self.keeps_latent else [])
+        downs = [get("dq")] + ([get("dkv")] if self.keeps_latent else []) + ([get("g")] if self.gate else [])
+        if self.sink:
+            self.sinks = placement.place(get("sink"), torch.float32)
         self.w_down, self.down_padded = stack_rows(downs, placement)
         self.q_norm = placement.place(get("dq.norm"))
         self.c_norm = placement.place(get("dkv.norm"), self.q_norm.dtype) if self.keeps_latent else None
@@ -131,6 +126,8 @@ class LatentAttention(Mixer):
         table = step.block_tables[cache.group]
         p = step.buffer("latent.down", (T, self.down_padded), torch.float32)
         ops.gemm(x, self.w_down, p, choices=step.choices)
+        g_col = Rq + (R + r if self.keeps_latent else 0)
+        extras = dict(sinks=self.sinks, gate=p[:, g_col:g_col + n] if self.gate else None)
         cq = step.buffer("latent.cq", (T, Rq), act)
         ops.latent_prepare(p, Rq, R if write_cache else 0, r, self.rot_dims, self.q_norm, self.c_norm, self.freq, self.mag,
                            step, table, cq, rows, self.eps)
@@ -150,7 +147,8 @@ class LatentAttention(Mixer):
             qa = step.buffer("latent.qa", (n, T, R), act)
             ops.latent.heads_gemm(qn, self.w_uk_t, qa)
             ol = ol.view(n, T, R)
-            ops.latent.latent_attention_mfma(qa, qr, rows, ol, step, table, n, R, self.scale, self.window, head_major=True)
+            ops.latent.latent_attention_mfma(qa, qr, rows, ol, step, table, n, R, self.scale, self.window, head_major=True,
+                                            **extras)
             oh = step.buffer("latent.oh", (n, T, dv), act)
             ops.latent.heads_gemm(ol, self.w_uv, oh)
             o = step.buffer("latent.o", (T, n * dv), act)
@@ -165,7 +163,8 @@ class LatentAttention(Mixer):
                 ops.latent.zero_(qr)
             if r:
                 ops.latent_q_rotate(q, self.freq, self.mag, step.positions, qr, n, d, r, self.rot_dims, 0)
-            ops.latent.latent_attention_mfma(qa, qr, rows, ol, step, table, n, R, self.scale, self.window, head_major=False)
+            ops.latent.latent_attention_mfma(qa, qr, rows, ol, step, table, n, R, self.scale, self.window, head_major=False,
+                                            **extras)
         else:
             qp = step.buffer("latent.qp", (T, n * D), act)
             if pad:
@@ -173,7 +172,7 @@ class LatentAttention(Mixer):
             ops.head_gemm(q, d + r, self.w_uk_t, qp, D, n, choices=step.choices)
             if r:
                 ops.latent_q_rotate(q, self.freq, self.mag, step.positions, qp, n, d, r, self.rot_dims, R)
-            ops.latent_attention(qp, rows, ol, step, table, n, R, self.scale, self.window)
+            ops.latent_attention(qp, rows, ol, step, table, n, R, self.scale, self.window, **extras)
         o = step.buffer("latent.o", (T, n * dv), act)
         ops.head_gemm(ol, R, self.w_uv, o, dv, n, choices=step.choices)
         ops.gemm(o, self.w_o, out, accumulate, fixed_order=step.fixed_order, choices=step.choices)

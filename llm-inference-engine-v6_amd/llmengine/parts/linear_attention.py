@@ -11,6 +11,14 @@ heads by silu(Wg x); then the output matrix.
 
 Kept per request: S, 32-bit, zero at admission. The decay (through its logarithm), the recurrence, the read-out norm
 and the gate are 32-bit. The recurrence is the delta rule's kernel without the read before the write.
+
+Lightning attention is the rule with one fixed decay a head, a constant of the model (`decay`):
+
+    S <- a S + k_t v_t^T;    o_t = S^T q_t
+
+with q, k and v the SiLU of their projections and no scale. The heads' reads side by side are divided by their common root
+mean square, multiplied by a weight of their whole size ("norm") and by sigmoid(Wg x); then the output matrix. It has kernels
+of its own, whose chunked form rests on the decay being the same for every token.
 """
 from __future__ import annotations
 
@@ -91,4 +99,46 @@ class GatedLinearAttention(ProjectedMixer):
         ops.gated_head_norm(read, self.norm_w, g_in, None, o, heads, vdim, self.eps, scale, activation="silu")
 
 
+class LightningAttention(ProjectedMixer):
+    def __init__(self, hidden_size: int, heads: int, dim: int, vdim: int, decay, eps: float):
+        self.hidden_size = int(hidden_size)
+        self.heads, self.dim, self.vdim = int(heads), int(dim), int(vdim)
+        self.decay, self.eps = tuple(float(a) for a in decay), float(eps)
+        if len(self.decay) != self.heads or not all(0.0 <= a <= 1.0 for a in self.decay):
+            raise ValueError(f"lightning attention: {self.heads} heads need as many decays between 0 and 1, got {list(self.decay)}")
+        self.out_width = self.heads * self.vdim
+
+    def input_names(self):
+        qk, hv = self.heads * self.dim, self.heads * self.vdim
+        return [("q", qk), ("k", qk), ("v", hv), ("g", hv)]
+
+    def output_name(self):
+        return "o"
+
+    def param_specs(self):
+        out = {name: ParamSpec((rows, self.hidden_size)) for name, rows in self.input_names()}
+        out.update({"norm": ParamSpec((self.out_width,), "norm"), "o": ParamSpec((self.hidden_size, self.out_width))})
+        return out
+
+    def refusals(self):
+        if self.dim > ops.lightning.MAX_DIM:
+            return [f"dim={self.dim}: the recurrence kernels take key sizes up to {ops.lightning.MAX_DIM}"]
+        return []
+
+    def cache_spec(self) -> CacheSpec:
+        return CacheSpec(state={"memory": ((self.heads, self.vdim, self.dim), torch.float32)})
+
+    def load_core(self, get: Getter, placement: Placement) -> None:
+        a = torch.tensor(self.decay, dtype=torch.float64)
+        self.decays = placement.place(torch.cat([a, torch.log(a)]).to(torch.float32), torch.float32)
+        self.norm_w = placement.place(get("norm"), torch.float32)
+
+    def core(self, p, step, cache, o, scale=1.0):
+        qk, hv = self.heads * self.dim, self.heads * self.vdim
+        read = step.buffer("lightning.read", (p.shape[0], hv), torch.float32)
+        ops.lightning.lightning(p, 0, qk, 2 * qk, self.decays, cache.state["memory"], step, read, self.heads, self.dim, self.vdim)
+        ops.lightning.joined_norm_gate(read, self.norm_w, p[:, 2 * qk + hv:2 * (qk + hv)], o, self.eps, scale)
+
+
 register_part("mixer", "gated_linear_attention", GatedLinearAttention)
+register_part("mixer", "lightning_attention", LightningAttention)

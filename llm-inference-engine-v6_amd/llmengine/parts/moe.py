@@ -8,6 +8,8 @@ first where `renormalize` is set. Expert e: down_e(act(gate_e x) * up_e x), no b
 "e<i>.gate", "e<i>.up", "e<i>.down"; the shared expert is a child part under "shared".
 
 `router="sigmoid"`: the scores are sigmoid(z), each expert's on its own, and the largest are chosen.
+`shared_gate`: the shared expert's result is multiplied by sigmoid(Wsg x), one number a token ("shared.sg" [1, hidden]; its
+row stands below the router's, whose product makes it).
 `weight_on="input"`: a chosen expert runs on weight * x and its result is added as it is (the weight is taken out of
 the expert's two input products: their 32-bit sums are multiplied by it in front of the activation).
 
@@ -25,6 +27,7 @@ import torch
 
 from .. import ops
 from .base import FeedForward, Getter, ParamSpec, Placement
+from .projected import stack_rows
 from .registry import register_part
 
 
@@ -34,7 +37,10 @@ class MixtureOfExperts(FeedForward):
     def __init__(self, hidden_size: int, intermediate_size: int, experts: int, top: int, scale: float = 1.0,
                  renormalize: bool = False, activation: str = "silu", shared: FeedForward | None = None,
                  expert_name: str = "e{}", router: str = "softmax", vocab_size: int = 0, limit: float = 0.0,
-                 weight_on: str = "output"):
+                 weight_on: str = "output", shared_gate: bool = False):
+        if shared_gate and (shared is None or router == "table"):
+            raise ValueError("mixture_of_experts: a gate on the shared expert needs one, and a router matrix")
+        self.shared_gate = bool(shared_gate)
         if router not in ("softmax", "sigmoid", "table"):
             raise ValueError(f"mixture_of_experts: router {router!r} is none of 'softmax', 'sigmoid' and 'table'")
         if weight_on not in ("output", "input"):
@@ -69,6 +75,8 @@ class MixtureOfExperts(FeedForward):
         H, FF = self.hidden_size, self.intermediate_size
         out = ({"router": ParamSpec((self.experts, H))} if self.router != "table"
                else {"table": ParamSpec((self.vocab_size, self.top), f"table:{self.experts}")})
+        if self.shared_gate:
+            out["shared.sg"] = ParamSpec((1, H))
         for e in range(self.experts):
             name = self.expert_name.format(e)
             out.update({f"{name}.gate": ParamSpec((FF, H)), f"{name}.up": ParamSpec((FF, H)), f"{name}.down": ParamSpec((H, FF))})
@@ -78,7 +86,10 @@ class MixtureOfExperts(FeedForward):
         # The router's matrix as the file has it: bfloat16 entries times the bfloat16 input are exact in 32-bit, so the
         # matrix-core product with its 32-bit sums is the 32-bit product; the 32-bit model widens it like everything else.
         if self.router != "table":
-            self.w_router = placement.place(get("router"))
+            if self.shared_gate:
+                self.w_router, self.route_columns = stack_rows([get("router"), get("shared.sg")], placement)
+            else:
+                self.w_router, self.route_columns = placement.place(get("router")), self.experts
         else:
             self.table = placement.place(get("table"))
             if int(self.table.min()) < 0 or int(self.table.max()) >= self.experts:
@@ -103,9 +114,9 @@ class MixtureOfExperts(FeedForward):
         if self.router == "table":
             ops.window.table_route(self.table, step.tokens, ids, wts)
         else:
-            logits = step.buffer("moe.logits", (T, E), f32)
+            logits = step.buffer("moe.logits", (T, self.route_columns), f32)
             ops.gemm(x, self.w_router, logits, choices=step.choices)
-            ops.moe_route(logits, top, self.scale, self.renormalize, ids, wts, scoring=self.router)
+            ops.moe_route(logits[:, :E], top, self.scale, self.renormalize, ids, wts, scoring=self.router)
         tile = ops.latent.moe_tile(x, self.w_gate_up, T * top, E, self.group, step.choices)
         cap = ops.moe_capacity(T * top, E, tile)
         place_pair, pair_place = step.buffer("moe.place_pair", (cap,), i32), step.buffer("moe.pair_place", (T * top,), i32)
@@ -135,10 +146,15 @@ class MixtureOfExperts(FeedForward):
                          step.choices)
         y = step.buffer("moe.y", (cap, H), f32)
         ops.moe_gemm(act, self.w_down, False, 0, y, place_pair, tile_expert, n_tiles, tile, 0, "silu", step.choices)
-        if self.shared is not None:
+        shared = dict()
+        if self.shared_gate:
+            rows = step.buffer("moe.shared", (T, H), f32)
+            self.shared.forward(x, step, rows, False)
+            shared = dict(shared=rows, shared_gate=logits[:, E:E + 1])
+        elif self.shared is not None:
             self.shared.forward(x, step, out, accumulate)
             accumulate = True
-        ops.moe_combine(y, pair_place, wts if self.weight_on == "output" else None, out, accumulate, top=top)
+        ops.moe_combine(y, pair_place, wts if self.weight_on == "output" else None, out, accumulate, top=top, **shared)
 
 
 register_part("feed_forward", "mixture_of_experts", MixtureOfExperts)

@@ -7,7 +7,16 @@
   (`rot_pairs="halves"`) or entry 2 i with entry 2 i + 1 ("neighbours"), by position * f_i with
   f_i = rot_base^(-2 i / rot_dims), optionally stretched by wavelength band (`rot_scaling`: factor, low, high,
   original: waves shorter than original / high stay, waves longer than original / low slow down by the factor,
-  between the two a linear blend in original / wavelength) or, with a factor alone, all slowed down by it;
+  between the two a linear blend in original / wavelength), over a ramp of pairs (factor, original, fast, slow: from the
+  pair that makes `fast` turns over `original` positions to the one that makes `slow`, and cos and sin times
+  0.1 ln(factor) + 1) or, with a factor alone, all slowed down by it;
+* `bias`: the query, key and value projections have biases ("q.b", "k.b", "v.b");
+* `conv_taps` > 0: a short causal convolution along the sequence on every channel of the projected queries, keys and values
+  ("q.conv", "k.conv", "v.conv" [channels, taps], no bias), behind the projections and in front of norm and rotation; the
+  last conv_taps - 1 projected rows of a request are kept in its state;
+* `v_mix`: values that mix with those of an earlier layer for the same token: "first" for the layer whose values the
+  others take, "mix" for those, v <- (1 - lambda) v + lambda v_first with a learned number ("vmix", which "first" does
+  not use); the mixed values are cached;
 * `qk_norm`: every query and key head is divided by its root mean square and multiplied by a weight over the
   head's entries ("q.norm", "k.norm", shared by all heads) before it is rotated; `qk_norm="unit"`: divided only, no
   weight (in front of the rotation or behind it: a rotation leaves a head's length as it is);
@@ -38,29 +47,13 @@ tokens make it a full cache.
 """
 from __future__ import annotations
 
-import math
-
 import torch
 
 from .. import ops
 from .base import PAGE, CacheSpec, Getter, ParamSpec, Placement
+from .frequencies import banded_frequencies, ramped_frequencies
 from .projected import ProjectedMixer
 from .registry import register_part
-
-
-def banded_frequencies(rot_dims: int, base: float, scaling: dict | None) -> torch.Tensor:
-    """[rot_dims / 2] float64: base^(-2 i / rot_dims), stretched by wavelength band where `scaling` is given."""
-    i = torch.arange(rot_dims // 2, dtype=torch.float64)
-    freq = torch.pow(torch.tensor(float(base), dtype=torch.float64), -2.0 * i / rot_dims)
-    if scaling and "low" not in scaling:
-        freq = freq / float(scaling["factor"])            # (every wave slowed down alike)
-    elif scaling:
-        factor, low, high, orig = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
-        wave = 2.0 * math.pi / freq
-        blend = (orig / wave - low) / (high - low) if high != low else torch.zeros_like(freq)
-        mixed = (1.0 - blend) * freq / factor + blend * freq
-        freq = torch.where(wave < orig / high, freq, torch.where(wave > orig / low, freq / factor, mixed))
-    return freq
 
 
 class WindowAttention(ProjectedMixer):
@@ -69,7 +62,7 @@ class WindowAttention(ProjectedMixer):
                  softcap: float = 0.0, values: str = "projected", gate: bool | str = False, maps: int = 1, qk_norm: bool | str = False,
                  eps: float = 1e-6, diff: float = 0.0, rot_pairs: str = "halves", sink: bool = False,
                  q_temp: tuple[float, int] | None = None, distance_bias: float = 0.0, own_kv: bool = True,
-                 cache_window: int | None = None, chunk: int = 0):
+                 cache_window: int | None = None, chunk: int = 0, bias: bool = False, conv_taps: int = 0, v_mix: str = ""):
         if heads % kv_heads:
             raise ValueError(f"{heads} query heads do not divide into {kv_heads} key/value heads")
         if rot_dims % 2 or not 0 <= rot_dims <= dim:
@@ -100,7 +93,14 @@ class WindowAttention(ProjectedMixer):
             raise ValueError("q_temp: the temperature steps every > 0 positions")
         if distance_bias < 0:
             raise ValueError("distance_bias must be >= 0")
+        if v_mix not in ("", "first", "mix"):
+            raise ValueError(f"v_mix {v_mix!r} is none of '', 'first' and 'mix'")
+        if (bias or conv_taps or v_mix) and (not own_kv or values != "projected"):
+            raise ValueError("biases, convolutions and mixed values go with queries, keys and values of the layer's own")
         self.hidden_size = int(hidden_size)
+        self.bias, self.conv_taps, self.v_mix = bool(bias), int(conv_taps), v_mix
+        self.mag, self.v_lambda = 1.0, None
+        self.qkv_bias = self.conv_w = None
         self.heads, self.kv_heads, self.dim, self.vdim = int(heads), int(kv_heads), int(dim), int(vdim)
         self.scale, self.softcap = float(scale), float(softcap)
         self.rot_dims, self.rot_base = int(rot_dims), float(rot_base)
@@ -117,6 +117,7 @@ class WindowAttention(ProjectedMixer):
         self.sinks = self.slopes = None
         self.eps, self.diff = float(eps), float(diff)
         self.out_width = self.heads * self.vdim
+        self.qkv_width = (self.heads + self.kv_heads) * self.maps * self.dim + self.kv_heads * self.vdim
         self.inv_freq: torch.Tensor | None = None
         self.wq = self.wk = None
         self.lam = 0.0
@@ -146,34 +147,56 @@ class WindowAttention(ProjectedMixer):
                 out["k.norm"] = ParamSpec((self.dim,), "norm")
         if self.sink:
             out["sink"] = ParamSpec((self.heads,))
+        for name, rows in self.input_names()[:3]:
+            if self.bias:
+                out[name + ".b"] = ParamSpec((rows,))
+            if self.conv_taps:
+                out[name + ".conv"] = ParamSpec((rows, self.conv_taps), "taps")
+        if self.v_mix:
+            out["vmix"] = ParamSpec(())
         if self.maps == 2:
             out.update({k: ParamSpec((self.dim,)) for k in ("lq1", "lk1", "lq2", "lk2")})
         return out
 
     def refusals(self):
+        out = []
         if max(self.dim, self.vdim) > ops.window.WINDOW_ATTENTION_MAX_ENTRIES:
-            return [f"dim={self.dim}, vdim={self.vdim}: the attention kernels hold heads of up to "
-                    f"{ops.window.WINDOW_ATTENTION_MAX_ENTRIES} entries"]
-        return []
+            out.append(f"dim={self.dim}, vdim={self.vdim}: the attention kernels hold heads of up to "
+                       f"{ops.window.WINDOW_ATTENTION_MAX_ENTRIES} entries")
+        if self.conv_taps > ops.recurrent.MAX_TAPS:
+            out.append(f"conv={self.conv_taps}: the convolution kernel takes up to {ops.recurrent.MAX_TAPS} taps")
+        return out
 
     def cache_spec(self) -> CacheSpec | None:
         if not self.own_kv:
             return None
         slides = self.cache_window > 0 and self.keep_first == 0
         kind, length = ("chunk", self.chunk) if self.chunk else ("window", self.cache_window) if slides else ("full", 0)
-        return CacheSpec(kind=kind, window=length,
+        state = {"conv": ((self.conv_taps - 1, self.qkv_width), torch.float32)} if self.conv_taps else {}
+        return CacheSpec(kind=kind, window=length, state=state,
                          paged={"k": (self.kv_heads * self.maps, PAGE, self.dim), "v": (self.kv_heads, self.vdim, PAGE)})
 
     def load_core(self, get: Getter, placement: Placement) -> None:
         f32 = torch.float32
         if self.rot_dims:
             # frequencies in 64-bit, stored in 32-bit; the angle is the kernel's 32-bit product with the position
-            self.inv_freq = placement.place(banded_frequencies(self.rot_dims, self.rot_base, self.rot_scaling).to(f32), f32)
+            if self.rot_scaling and "fast" in self.rot_scaling:
+                freq, self.mag = ramped_frequencies(self.rot_dims, self.rot_base, self.rot_scaling)
+            else:
+                freq = banded_frequencies(self.rot_dims, self.rot_base, self.rot_scaling)
+            self.inv_freq = placement.place(freq.to(f32), f32)
         if self.norm_weights:
             self.wq = placement.place(get("q.norm"), f32)
             self.wk = placement.place(get("k.norm"), f32) if self.own_kv else None
         if self.sink:
             self.sinks = placement.place(get("sink"), f32)
+        if self.bias:
+            self.qkv_bias = placement.place(torch.cat([get(f"{c}.b").to(f32) for c in "qkv"]), f32)
+        if self.conv_taps:
+            self.conv_w = placement.place(torch.cat([get(f"{c}.conv").to(f32) for c in "qkv"]), f32)
+        if self.v_mix:
+            lam = float(get("vmix").to(f32))
+            self.v_lambda = lam if self.v_mix == "mix" else None
         if self.distance_bias:
             h = torch.arange(1, self.heads + 1, dtype=torch.float64)
             self.slopes = placement.place(torch.pow(2.0, -self.distance_bias * h / self.heads).to(f32), f32)
@@ -196,12 +219,23 @@ class WindowAttention(ProjectedMixer):
         k_cache, v_cache = cache.paged["k"], cache.paged["v"]
         q = step.buffer("window_attention.q", (T, nq * dim), step.act_dtype)
         unit = self.qk_norm and not self.norm_weights
+        qkv = p
+        if self.conv_taps:
+            qkv = step.buffer("window_attention.qkv", (T, g_col), torch.float32)
+            ops.short_conv(p[:, :g_col], self.conv_w, None, cache.state["conv"], step, qkv, silu=False, in_bias=self.qkv_bias)
+        elif self.bias:
+            qkv = step.buffer("window_attention.qkv", (T, g_col), torch.float32)
+            ops.copy_cols(p[:, :g_col], qkv)
+            ops.window.add_row_bias(qkv, self.qkv_bias)
+        # (the values that later layers mix with stay where they are until the step ends)
+        v_first = step.buffer("window_attention.first_values", (T, g * vdim), torch.float32) if self.v_mix else None
         if own:
-            ops.window.qk_prepare(p, step, table, q, k_cache, v_cache, nq, k_col, v_col, self.inv_freq, self.rot_dims,
-                                  self.wq, self.wk, self.eps, self.rot_pairs, self.q_temp, unit_norm=unit)
+            ops.window.qk_prepare(qkv, step, table, q, k_cache, v_cache, nq, k_col, v_col, self.inv_freq, self.rot_dims,
+                                  self.wq, self.wk, self.eps, self.rot_pairs, self.q_temp, unit_norm=unit, mag=self.mag,
+                                  v_first=v_first, v_mix=self.v_lambda)
         else:
             ops.window.qk_prepare(p, step, None, q, None, None, nq, 0, None, self.inv_freq, self.rot_dims, self.wq, None,
-                                  self.eps, self.rot_pairs, self.q_temp, dk=dim, unit_norm=unit)
+                                  self.eps, self.rot_pairs, self.q_temp, dk=dim, unit_norm=unit, mag=self.mag)
         # what is done with the runs' parts; where the keys are in one run the attention kernel may do it itself
         if M == 2:
             finish = dict(out=o, mode="difference", lam=self.lam, eps=self.eps, out_scale=(1.0 - self.diff) * scale)
