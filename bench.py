@@ -24,6 +24,8 @@ with biases and clamped experts chosen by a table, a stretch of layers that runs
 `--design zapolorn` the Zapolorn design (sublayers normed behind; windowed attention with sinks and head gates, one layer in
 three reading the keys of the layer in front; attention with a bias by distance beside a gated linear attention; dense
 feed-forwards and experts that weigh their input),
+`--design diporax` the Diporax design (sublayers normed behind; lightning attention, softmax attention with short convolutions
+and mixed values, latent attention with sinks, every layer with experts and an input of its own from the token's id);
 `--design lukupel` the Lukupel design (sublayers normed behind; a matrix memory with exponential gates, and attention within
 chunks of the sequence; feed-forwards with a squared rectifier).
 
@@ -188,7 +190,28 @@ def lukupel_at(width: int, ff: int, heads: int, layers: int, vocab: int, only: s
             "layers": [kinds[only or ("mlstm", "chunked", "chunked")[i % 3]] for i in range(layers)]}
 
 
-DESIGNS = {"rilonex": rilonex_at, "bidirax": bidirax_at, "zetonex": zetonex_at, "zapolorn": zapolorn_at, "lukupel": lukupel_at}
+def diporax_at(width: int, ff: int, heads: int, layers: int, vocab: int, only: str = "") -> dict:
+    """Diporax layers of a Llama layer's width, heads and active feed-forward size: lightning attention (half as many heads,
+    keys and values of 128), softmax attention over everything before (heads of 64, a quarter as many key heads, biases and
+    convolutions of 4 taps, half of a head rotated, capped scores, mixed values) and latent attention (a latent of 256 and a
+    rotated part of 32, a sink and a gate per head), every one with 16 experts (2 a token, a quarter of the feed-forward size
+    each, beside a gated shared one of half of it) and an eighth of the width from the per-token table."""
+    moe = {"kind": "moe", "router": {"experts": 16, "top": 2}, "expert": {"ff": ff // 4}, "shared": {"ff": ff // 2}}
+    n = max(1, heads // 2)
+    rot = {"base": 500000.0, "dims": 32, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}
+    kinds = {
+        "lightning": {"type": "lightning", "mixer": {"heads": n, "dim": 128, "vdim": 128,
+                                                     "decay": [1.0 - 2.0 ** (-1.0 - 8.0 * i / n) for i in range(n)]}, "mlp": moe},
+        "full": {"type": "attention", "mixer": {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 64, "vdim": 64, "scale": 0.125,
+                                                "conv": 4, "softcap": 30.0, "v_mix": True, "rot": rot}, "mlp": moe},
+        "latent": {"type": "latent_attention", "mixer": {"heads": heads, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": 256,
+                                                         "q_rank": width // 2, "scale": 96 ** -0.5, "rot": rot}, "mlp": moe},
+    }
+    return {"architecture": "Diporax", "vocab": vocab, "width": width, "norm": {"eps": 1e-6}, "token_side": {"dim": width // 8},
+            "layers": [kinds[only or ("lightning", "full", "latent")[i % 3]] for i in range(layers)]}
+
+
+DESIGNS = {"diporax": diporax_at, "rilonex": rilonex_at, "bidirax": bidirax_at, "zetonex": zetonex_at, "zapolorn": zapolorn_at, "lukupel": lukupel_at}
 
 
 def design(args) -> int:
@@ -449,9 +472,9 @@ def main() -> int:
     ap.add_argument("--design", default="rilonex", choices=sorted(DESIGNS),
                     help="design: which design runs beside Llama")
     ap.add_argument("--design-only", default="", choices=["", "rglru", "channel_delta", "parallel", "rotated", "windowed", "differential", "gated", "mlstm",
-                                                             "chunked"],
+                                                             "chunked", "lightning", "full", "latent"],
                     help="design: a model of this kind of layer only (the first three Rilonex, the next two Bidirax, two "
-                         "more Zetonex, the last two Lukupel; Zapolorn: windowed or parallel)")
+                         "more Zetonex, two Lukupel, the last three Diporax; Zapolorn: windowed or parallel)")
     ap.add_argument("--design-skip-llama", action="store_true", help="design: time the design alone")
     ap.add_argument("--portion", type=int, default=256, help="portion: prompt tokens a step")
     ap.add_argument("--decode-len", type=int, default=700, help="mixed: tokens of the shortest decoding request "

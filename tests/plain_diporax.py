@@ -156,7 +156,7 @@ def attention(x, w, m, eps, values):
     v = proj["v"].view(T, g, dv)
     if m.get("v_mix"):
         if "first" in values:
-            v = mix_values(v, values["first"], w["vmix"])
+            v = mix_values(v, values["first"].reshape(v.shape), w["vmix"])        # (entry by entry, however they are cut into heads)
         else:
             values["first"] = v
     o = attend(q, k, v, m["scale"], float(m.get("softcap") or 0.0))
