@@ -113,6 +113,8 @@ struct Groups {
     const int* row_index = nullptr;
     int gather_div = 1;
     int rows_per_group = 0, tiles_per_group = 1;
+    int rows_out = 0;           // heads: `out` is [rows_per_group, groups * N], the groups' results side by side
+    int n_groups = 1;
     long w_stride = 0;          // elements
     unsigned a_bytes = 0;       // of the whole of `a`, where rows are gathered
 };
@@ -193,8 +195,11 @@ __device__ __forceinline__ void tile_epilogue(f32x4 (&acc)[WMT][WNT], unsigned c
                                               int M, int N, int m0, int n0, int wm, int wn, int tid, int r, int q,
                                               const QkvTarget& qt = QkvTarget{},
                                               const AddendsAhead<WR * 16 * WMT, WC * 16 * WNT, 64 * WR * WC>& ahead = {},
-                                              const RowPlace& place = RowPlace{}, const GateExtra& gx = GateExtra{}) {
+                                              const RowPlace& place = RowPlace{}, const GateExtra& gx = GateExtra{},
+                                              int stored_ld = 0) {
     constexpr int BM = WR * 16 * WMT, BN = WC * 16 * WNT, NT = 64 * WR * WC;
+    // (a result stored in bfloat16 may lie in rows further apart than its columns: heads side by side)
+    const size_t ld16 = static_cast<size_t>(stored_ld > 0 ? stored_ld : N);
 
     constexpr int SS = BN + 4;                           // floats per staged row
     // A tile that is larger than the LDS goes through it in 2 or 4 passes of whole wavefront rows.
@@ -332,7 +337,7 @@ __device__ __forceinline__ void tile_epilogue(f32x4 (&acc)[WMT][WNT], unsigned c
                 bf16x8 o;
 #pragma unroll
                 for (int e = 0; e < 8; ++e) o[e] = static_cast<__bf16>(stored_value<MODE>(sp[e]));
-                *reinterpret_cast<bf16x8*>(static_cast<bf16*>(out) + static_cast<size_t>(m) * N + n) = o;
+                *reinterpret_cast<bf16x8*>(static_cast<bf16*>(out) + static_cast<size_t>(m) * ld16 + n) = o;
             }
         } else if (MODE == kAddF32 && PASSES == 1 && AHEAD) {
             constexpr int PER_ROW = BN / 4;
@@ -401,7 +406,7 @@ __device__ __forceinline__ void tile_epilogue(f32x4 (&acc)[WMT][WNT], unsigned c
                     if (MODE == kStoreF32) static_cast<float*>(out)[idx] = v;
                     else if (MODE == kAddF32) static_cast<float*>(out)[idx] += v;
                     else if (MODE == kAtomicF32) atomicAdd(static_cast<float*>(out) + idx, v);
-                    else static_cast<bf16*>(out)[idx] = static_cast<bf16>(stored_value<MODE>(v));
+                    else static_cast<bf16*>(out)[static_cast<size_t>(m) * ld16 + n] = static_cast<bf16>(stored_value<MODE>(v));
                 }
             }
         }
@@ -439,7 +444,7 @@ __global__ __launch_bounds__(256, 2) void gemm_tile_kernel(const bf16* __restric
     const int gsize = (tiles_m - first_m < GROUP) ? tiles_m - first_m : GROUP;
     const int tm = first_m + (pid % per_group) % gsize;
     const int tn = (pid % per_group) / gsize;
-    int m0 = tm * BM;
+    int m0 = tm * BM, stored_ld = 0;
     const int n0 = tn * BN;
     if (GROUPED) {
         if (gr.n_tiles != nullptr && tm >= gr.n_tiles[0]) return;
@@ -450,6 +455,10 @@ __global__ __launch_bounds__(256, 2) void gemm_tile_kernel(const bf16* __restric
             group = tm / gr.tiles_per_group;
             m0 = group * gr.rows_per_group + (tm % gr.tiles_per_group) * BM;
             M = (group + 1) * gr.rows_per_group;
+            if (gr.rows_out) {
+                stored_ld = gr.n_groups * N;
+                out = static_cast<bf16*>(out) + static_cast<long>(group) * N - static_cast<long>(group) * gr.rows_per_group * stored_ld;
+            }
         }
         w += static_cast<size_t>(group) * gr.w_stride;
     }
@@ -636,7 +645,7 @@ __global__ __launch_bounds__(256, 2) void gemm_tile_kernel(const bf16* __restric
     if (AHEAD && N % 8 == 0) addends.load(out, M, N, m0, n0, tid);
     __syncthreads();                                  // the epilogue reuses the slabs' LDS
     tile_epilogue<WMT, WNT, MODE, tile_lds_bytes<WMT, WNT>(), 2, 2, AHEAD>(acc, lds_raw, out, M, N, m0, n0, wm, wn, tid, r, q,
-                                                                           qt, addends, place, gx);
+                                                                           qt, addends, place, gx, stored_ld);
 }
 
 // ----------------------------------------------------------------------------------------
@@ -1230,11 +1239,13 @@ extern "C" int llme_gemm_bf16(const void* a, const void* w, void* out, int out_d
 // Products in groups on the tile kernel (see Groups). a [a_rows, K], w [groups, N, K] row-major, both bfloat16.
 // Experts (tile_group given): `out` has max_tiles * tile rows, row tile t belongs to expert tile_group[t] and exists if
 // t < n_tiles[0]; row m of a tile is row row_index[m] / gather_div of `a` (row_index null: row m itself; negative: zeros).
-// Heads (tile_group null): group g owns rows g * rows_per_group .. of `a` and of `out`.
+// Heads (tile_group null): group g owns rows g * rows_per_group .. of `a` and of `out`; rows_out (bfloat16): `out` is
+// [rows_per_group, groups * N] instead, the groups' results side by side.
 // gated: w holds gate and up rows interleaved in groups of 16, out [.., N / 2] = silu(gate) * up. tile: 64 or 128 rows.
 extern "C" int llme_gemm_bf16_grouped(const void* a, const void* w, void* out, int out_dtype, int gated, int N, int K, int tile,
                                       int max_tiles, const int* tile_group, const int* n_tiles, const int* row_index,
-                                      int gather_div, long a_rows, int groups, int rows_per_group, hipStream_t stream) {
+                                      int gather_div, long a_rows, int groups, int rows_per_group, int rows_out, hipStream_t stream) {
+    if (rows_out && (tile_group != nullptr || gated || out_dtype != kBF16)) return kErrBadArgument;
     if (N <= 0 || groups <= 0) return 0;
     if (K <= 0 || K % 8 != 0 || K >= (1 << 23) || (tile != 64 && tile != 128)) return kErrUnsupported;
     if (out_dtype != kF32 && out_dtype != kBF16) return kErrBadArgument;
@@ -1255,6 +1266,8 @@ extern "C" int llme_gemm_bf16_grouped(const void* a, const void* w, void* out, i
     } else {
         if (rows_per_group <= 0) return 0;
         gr.rows_per_group = rows_per_group;
+        gr.rows_out = rows_out;
+        gr.n_groups = groups;
         gr.tiles_per_group = (rows_per_group + tile - 1) / tile;
         tiles_m = groups * gr.tiles_per_group;
         M = groups * rows_per_group;
@@ -1293,7 +1306,7 @@ extern "C" int llme_gemm_bf16_grouped_gated_extra(const void* a, const void* w, 
     t_gate_extra.row_pair = pair_scale != nullptr ? row_index : nullptr;
     t_gate_extra.pair_scale = pair_scale;
     const int rc = llme_gemm_bf16_grouped(a, w, out, kBF16, 4, N, K, tile, max_tiles, tile_group, n_tiles, row_index, gather_div,
-                                          a_rows, groups, 0, stream);
+                                          a_rows, groups, 0, 0, stream);
     t_gate_extra = GateExtra{};
     return rc;
 }

@@ -89,7 +89,8 @@ __global__ __launch_bounds__(256) void latent_attention_mfma_kernel(LatentArgs a
     const int s = blockIdx.y, z = blockIdx.z;
     const int first_tok = a.q_start[s], n_tok = a.q_start[s + 1] - first_tok;
     const int pairs = n_tok * a.n;
-    const int p0 = blockIdx.x * 64;
+    // (the last rows, which see the most keys, go first: the short ones fill in behind them)
+    const int p0 = (gridDim.x - 1 - blockIdx.x) * 64;
     if (p0 >= pairs) return;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int r16 = lane & 15, g = lane >> 4;
@@ -334,16 +335,6 @@ __global__ void latent_q_split_kernel(const bf16* __restrict__ q, const float* _
     dst[1] = static_cast<bf16>(v * cs + u * sn);
 }
 
-// o [n, T, c] -> out [T, n c]
-__global__ void heads_to_rows_kernel(const bf16* __restrict__ o, bf16* __restrict__ out, int T, int n, int c, size_t total) {
-    const size_t idx = static_cast<size_t>(blockIdx.x) * 256 + threadIdx.x;
-    if (idx >= total) return;
-    const int e = static_cast<int>(idx % c);
-    const size_t th = idx / c;
-    const int h = static_cast<int>(th % n), t = static_cast<int>(th / n);
-    out[idx] = o[(static_cast<size_t>(h) * T + t) * c + e];
-}
-
 template <int DC, int RC>
 static int launch_latent(const LatentArgs& a, int max_new, int n_seq, hipStream_t stream) {
     const int D = a.R + a.r;
@@ -398,14 +389,6 @@ extern "C" int llme_latent_q_split(const void* q, const float* freq, float mag, 
     hipLaunchKernelGGL(latent_q_split_kernel, dim3(static_cast<unsigned>((total + 255) / 256)), dim3(256), 0, stream,
                        static_cast<const bf16*>(q), freq, mag, positions, static_cast<bf16*>(qn), static_cast<bf16*>(qr), T, n, d,
                        r, rd, total);
-    return launch_status();
-}
-
-extern "C" int llme_heads_to_rows(const void* o, void* out, int T, int n, int c, hipStream_t stream) {
-    if (T <= 0) return 0;
-    const size_t total = static_cast<size_t>(T) * n * c;
-    hipLaunchKernelGGL(heads_to_rows_kernel, dim3(static_cast<unsigned>((total + 255) / 256)), dim3(256), 0, stream,
-                       static_cast<const bf16*>(o), static_cast<bf16*>(out), T, n, c, total);
     return launch_status();
 }
 

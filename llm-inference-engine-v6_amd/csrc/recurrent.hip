@@ -44,6 +44,79 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const float* __restrict
     out[static_cast<size_t>(t) * ld_out + c] = act == 1 ? siluf_(acc) : acc;
 }
 
+// The same for steps of many rows, K taps known: a thread makes four neighbouring channels of eight rows, the last K - 1 inputs
+// in registers as it walks them, so that an input is read from memory once and not once a tap. All sizes and strides in whole
+// groups of four.
+constexpr int kConvRows = 8;
+
+template <int K>
+__global__ __launch_bounds__(256) void short_conv_rows_kernel(const float* __restrict__ in, int ld_in, const float* __restrict__ w,
+                                                              const float* __restrict__ bias, const float* __restrict__ in_bias,
+                                                              const float* __restrict__ tail, const int* __restrict__ seq_idx,
+                                                              const int* __restrict__ q_start, const int* __restrict__ slots,
+                                                              float* __restrict__ out, int ld_out, int T, int C, int act) {
+    const int c = (blockIdx.x * 256 + threadIdx.x) * 4;
+    if (c >= C) return;
+    const int t0 = blockIdx.y * kConvRows, t1 = min(t0 + kConvRows, T);
+    auto load4 = [](const float* p, float (&v)[4]) {
+        const float4 x = *reinterpret_cast<const float4*>(p);
+        v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
+    };
+    float wt[4][K], b[4] = {0.f, 0.f, 0.f, 0.f}, ib[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int j = 0; j < K; ++j) wt[e][j] = w[static_cast<size_t>(c + e) * K + j];
+    if (bias != nullptr) load4(bias + c, b);
+    if (in_bias != nullptr) load4(in_bias + c, ib);
+    float x[kConvRows][4];
+#pragma unroll
+    for (int i = 0; i < kConvRows; ++i)
+        if (t0 + i < t1) {
+            load4(in + static_cast<size_t>(t0 + i) * ld_in + c, x[i]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[i][e] += ib[e];
+        }
+    int s = seq_idx[t0];
+    int first = q_start[s], next = q_start[s + 1];
+    float win[K - 1][4];                                    // the inputs of the K - 1 rows in front of the one at hand, oldest first
+#pragma unroll
+    for (int i = 0; i < K - 1; ++i) {
+        const int r = t0 - (K - 1) + i;
+        if (r >= first) {
+            load4(in + static_cast<size_t>(r) * ld_in + c, win[i]);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) win[i][e] += ib[e];
+        } else {
+            load4(tail + (static_cast<size_t>(slots[s]) * (K - 1) + K - 1 + (r - first)) * C + c, win[i]);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < kConvRows; ++i) {
+        const int t = t0 + i;
+        if (t >= t1) break;
+        if (t >= next) {                                    // another request's first row: what lies in front of it is in its tail
+            s = seq_idx[t];
+            next = q_start[s + 1];
+#pragma unroll
+            for (int j = 0; j < K - 1; ++j) load4(tail + (static_cast<size_t>(slots[s]) * (K - 1) + j) * C + c, win[j]);
+        }
+        float y[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            float acc = b[e];
+#pragma unroll
+            for (int j = 0; j < K - 1; ++j) acc += wt[e][j] * win[j][e];
+            acc += wt[e][K - 1] * x[i][e];
+            y[e] = act == 1 ? siluf_(acc) : acc;
+#pragma unroll
+            for (int j = 0; j + 1 < K - 1; ++j) win[j][e] = win[j + 1][e];
+            win[K - 2][e] = x[i][e];
+        }
+        *reinterpret_cast<float4*>(out + static_cast<size_t>(t) * ld_out + c) = float4{y[0], y[1], y[2], y[3]};
+    }
+}
+
 // A step in which every request brings one row (decoding): the convolution and the tail's move in one kernel. A thread
 // reads its channel's tail, makes the row's output and stores the tail moved on by the row.
 __global__ __launch_bounds__(256) void short_conv_single_kernel(const float* __restrict__ in, int ld_in, const float* __restrict__ w,
@@ -607,6 +680,20 @@ extern "C" int llme_short_conv(const void* in, int ld_in, const void* w, const v
             static_cast<const int*>(slots), static_cast<float*>(out), ld_out, C, K, act);
         return launch_status();
     }
+    auto aligned = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
+    if (K >= 2 && K <= 4 && T >= 32 && C % 4 == 0 && ld_in % 4 == 0 && ld_out % 4 == 0 && aligned(in) && aligned(bias) && aligned(in_bias) &&
+        aligned(tail) && aligned(out)) {
+        const dim3 rows_grid((C / 4 + 255) / 256, (T + kConvRows - 1) / kConvRows);
+#define LLME_CONV_ROWS(K_)                                                                                                            \
+    short_conv_rows_kernel<K_><<<rows_grid, 256, 0, stream>>>(                                                                        \
+        static_cast<const float*>(in), ld_in, static_cast<const float*>(w), static_cast<const float*>(bias),                          \
+        static_cast<const float*>(in_bias), static_cast<const float*>(tail), static_cast<const int*>(seq_idx),                        \
+        static_cast<const int*>(q_start), static_cast<const int*>(slots), static_cast<float*>(out), ld_out, T, C, act)
+        if (K == 2) LLME_CONV_ROWS(2);
+        else if (K == 3) LLME_CONV_ROWS(3);
+        else LLME_CONV_ROWS(4);
+#undef LLME_CONV_ROWS
+    } else
     short_conv_kernel<<<grid, 256, 0, stream>>>(
         static_cast<const float*>(in), ld_in, static_cast<const float*>(w), static_cast<const float*>(bias),
         static_cast<const float*>(in_bias), static_cast<const float*>(tail), static_cast<const int*>(seq_idx),

@@ -32,6 +32,46 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(const TT* __restrict__ 
     for (int i = threadIdx.x; i < H; i += 256) out[static_cast<size_t>(t) * H + i] = (to_float(w[i]) * row[i]) * inv;
 }
 
+// The same for rows of up to 8,192 entries in whole pieces of eight, which stay in registers (NV pieces a thread); in either layout
+// a piece's entries lie together.
+template <typename TT, typename TW, int NV>
+__global__ __launch_bounds__(256) void embed_norm_vec_kernel(const TT* __restrict__ table, const int* __restrict__ tokens,
+                                                             const TW* __restrict__ w, float* __restrict__ out, int H, float eps, int blocked) {
+    __shared__ float scratch[4];
+    struct alignas(16) TablePiece { TT x[8]; };
+    struct alignas(16) WeightPiece { TW x[8]; };
+    const int t = blockIdx.x, id = tokens[t];
+    const TT* src = blocked ? table + static_cast<size_t>(id / 16) * 16 * H + (id % 16) * 8 : table + static_cast<size_t>(id) * H;
+    float v[NV][8], wv[NV][8], ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int j = threadIdx.x + 256 * k;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[k][e] = wv[k][e] = 0.f;
+        if (j * 8 >= H) continue;
+        const TablePiece p = *reinterpret_cast<const TablePiece*>(src + (blocked ? static_cast<size_t>(j / 4) * 512 + (j % 4) * 128 : static_cast<size_t>(j) * 8));
+        const WeightPiece q = *reinterpret_cast<const WeightPiece*>(w + j * 8);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+            v[k][e] = to_float(p.x[e]);
+            wv[k][e] = to_float(q.x[e]);
+            ss = fmaf(v[k][e], v[k][e], ss);
+        }
+    }
+    const float inv = 1.0f / sqrtf(block_sum(ss, scratch, 4) / static_cast<float>(H) + eps);
+#pragma unroll
+    for (int k = 0; k < NV; ++k) {
+        const int j = threadIdx.x + 256 * k;
+        if (j * 8 >= H) continue;
+        float y[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) y[e] = (wv[k][e] * v[k][e]) * inv;
+        float4* dst = reinterpret_cast<float4*>(out + static_cast<size_t>(t) * H + j * 8);
+        dst[0] = float4{y[0], y[1], y[2], y[3]};
+        dst[1] = float4{y[4], y[5], y[6], y[7]};
+    }
+}
+
 template <typename TT, typename TO>
 __global__ __launch_bounds__(256) void token_gate_kernel(const float* __restrict__ z, int ld_z, const TT* __restrict__ table, int ld_table,
                                                          int col, const int* __restrict__ tokens, TO* __restrict__ out, int n, size_t total) {
@@ -52,9 +92,21 @@ extern "C" int llme_embed_norm(const void* table, int table_dtype, const int* to
     if (H <= 0 || H > 15000) return kErrUnsupported;
     if (blocked && (table_dtype != kBF16 || H % 32 != 0)) return kErrUnsupported;
     const size_t lds = static_cast<size_t>(H) * sizeof(float);
-#define LLME_EN(TT, TW)                                                                                                     \
-    hipLaunchKernelGGL((embed_norm_kernel<TT, TW>), dim3(T), dim3(256), lds, stream, static_cast<const TT*>(table), tokens, \
+    const bool vec = H % 8 == 0 && H <= 8192 && reinterpret_cast<uintptr_t>(table) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0 &&
+                     reinterpret_cast<uintptr_t>(out) % 16 == 0;
+    const int nv = !vec ? 0 : H <= 2048 ? 1 : H <= 4096 ? 2 : 4;
+#define LLME_EN_V(TT, TW, NV)                                                                                                        \
+    hipLaunchKernelGGL((embed_norm_vec_kernel<TT, TW, NV>), dim3(T), dim3(256), 0, stream, static_cast<const TT*>(table), tokens,     \
                        static_cast<const TW*>(w), out, H, eps, blocked)
+#define LLME_EN(TT, TW)                                                                                                             \
+    do {                                                                                                                            \
+        if (nv == 1) LLME_EN_V(TT, TW, 1);                                                                                          \
+        else if (nv == 2) LLME_EN_V(TT, TW, 2);                                                                                     \
+        else if (nv == 4) LLME_EN_V(TT, TW, 4);                                                                                     \
+        else                                                                                                                        \
+            hipLaunchKernelGGL((embed_norm_kernel<TT, TW>), dim3(T), dim3(256), lds, stream, static_cast<const TT*>(table), tokens, \
+                               static_cast<const TW*>(w), out, H, eps, blocked);                                                    \
+    } while (0)
     switch (table_dtype * 2 + w_dtype) {
         case 0: LLME_EN(float, float); break;
         case 1: LLME_EN(float, bf16); break;
@@ -63,6 +115,7 @@ extern "C" int llme_embed_norm(const void* table, int table_dtype, const int* to
         default: return kErrBadArgument;
     }
 #undef LLME_EN
+#undef LLME_EN_V
     return launch_status();
 }
 

@@ -171,7 +171,6 @@ def latent_attention(qp: torch.Tensor, cache: torch.Tensor, out: torch.Tensor, s
 declare("llme_latent_attention_mfma", [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _i, _i, _f, _i, _i,
                                        _l, _l, _l, _l, _vp, _vp, _i, _vp])
 declare("llme_latent_q_split", [_vp, _vp, _f, _vp, _vp, _vp, _i, _i, _i, _i, _i, _vp])
-declare("llme_heads_to_rows", [_vp, _vp, _i, _i, _i, _vp])
 LATENT_MFMA_MAX_ROW, LATENT_MFMA_MAX_RANK = 576, 512
 
 
@@ -241,16 +240,8 @@ def latent_q_split(q: torch.Tensor, freq: torch.Tensor | None, mag: float, posit
                                        ptr(qr) if rot else None, T, heads, dim, rot, rot_dims, stream()), "latent_q_split")
 
 
-def heads_to_rows(o: torch.Tensor, out: torch.Tensor) -> None:
-    """o [heads, T, c] -> out [T, heads * c]."""
-    require(o, "o", torch.bfloat16, (None, None, None))
-    n, T, c = o.shape
-    require(out, "out", torch.bfloat16, (T, n * c))
-    check(entry("llme_heads_to_rows")(ptr(o), ptr(out), T, n, c, stream()), "heads_to_rows")
-
-
 # --- products in groups on the matrix cores -------------------------------------------------
-declare("llme_gemm_bf16_grouped", [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp, _vp, _vp, _i, _l, _i, _i, _vp])
+declare("llme_gemm_bf16_grouped", [_vp, _vp, _vp, _i, _i, _i, _i, _i, _i, _vp, _vp, _vp, _i, _l, _i, _i, _i, _vp])
 
 
 def _grouped_fits(a: torch.Tensor, w: torch.Tensor, choices) -> bool:
@@ -264,26 +255,39 @@ def heads_gemm_fits(a: torch.Tensor, w: torch.Tensor, choices=None) -> bool:
 
 
 def heads_gemm(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor) -> None:
-    """out[h] = a[h] w[h]^T for a [heads, T, K], w [heads, N, K], out [heads, T, N], all bfloat16: the matrix-core tile
-    kernel with a matrix per group of row tiles."""
+    """out[h] = a[h] w[h]^T for a [heads, T, K], w [heads, N, K], out [heads, T, N] or, the heads side by side,
+    [T, heads N], all bfloat16: the matrix-core tile kernel with a matrix per group of row tiles."""
     require(a, "a", torch.bfloat16, (None, None, None))
     n, T, K = a.shape
     require(w, "w", torch.bfloat16, (n, None, K))
     N = w.shape[1]
-    require(out, "out", torch.bfloat16, (n, T, N))
+    require(out, "out", torch.bfloat16, (n, T, N) if out.dim() == 3 else (T, n * N))
     tile = 128 if T >= 512 else 64
     check(entry("llme_gemm_bf16_grouped")(ptr(a), ptr(w), ptr(out), code(out.dtype), 0, N, K, tile, 0, None, None, None, 1,
-                                          n * T, n, T, stream()), "heads_gemm")
+                                          n * T, n, T, 1 if out.dim() == 2 else 0, stream()), "heads_gemm")
 
 
 # --- mixture of experts ----------------------------------------------------------------
 MOE_FAST_TILES = (64, 128)
+MOE_COMBINE_NORM_MAX = 8192     # entries of a row that moe_combine_norm holds
+MOE_FEW_PAIRS = 4               # pairs an expert, on average, up to which tiles of 16 rows are taken on the matrix cores
+declare("llme_gemm_few_gated", [_vp, _vp, _vp, _i, _i, _i, _i, _i, _vp])
+declare("llme_gemm_few_token_gate", [_vp, _vp, _vp, _i, _i, _i, _i, _vp, _i, _i, _vp, _vp])
+declare("llme_gemm_few_grouped", [_vp, _vp, _vp, _i, _i, _i, _i, _i, _vp, _vp, _vp, _i, _vp, _vp])
+
+
+def moe_few_rows(tile: int, a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gated: bool, group: int, activation: str, choices) -> bool:
+    """Whether the matrix-core kernel for tiles of 16 rows takes an experts' product."""
+    from .recurrent import GATE_ACTIVATIONS
+    return (tile == MOE_TILE and _grouped_fits(a, w, choices)
+            and (group == 16 and activation in GATE_ACTIVATIONS and out.dtype == torch.bfloat16 if gated else out.dtype == torch.float32))
 
 
 def moe_tile(x: torch.Tensor, w: torch.Tensor, pairs: int, experts: int, group: int, choices=None) -> int:
-    """Rows of a tile for a step's grouped products: 16 for the plain-precision kernel; 64 or 128 on the matrix cores
-    (bfloat16, gate and up rows interleaved in groups of 16)."""
-    if not _grouped_fits(x, w, choices) or group != 16:
+    """Rows of a tile for a step's grouped products: 16 for the plain-precision kernel and, on the matrix cores, for few rows
+    an expert (decoding: the weights are streamed); otherwise 64 or 128 on the matrix cores (bfloat16, gate and up rows
+    interleaved in groups of 16)."""
+    if not _grouped_fits(x, w, choices) or group != 16 or pairs <= MOE_FEW_PAIRS * experts:
         return MOE_TILE
     return 128 if pairs >= 128 * experts else 64
 
@@ -324,8 +328,8 @@ def moe_plan(ids: torch.Tensor, experts: int, tile: int, place_pair: torch.Tenso
 
 def moe_gemm(a: torch.Tensor, w: torch.Tensor, gated: bool, group: int, out: torch.Tensor, place_pair: torch.Tensor,
              tile_expert: torch.Tensor, n_tiles: torch.Tensor, tile: int, gather_div: int, activation: str = "silu",
-             choices=None) -> None:
-    """Per place: out[place] = w[expert] a[row]; gated: act(gate a) * (up a), w [experts, 2 N, K] holding gate and up rows in
+             choices=None, pairs: int = 0, pair_scale: torch.Tensor | None = None) -> None:
+    """pairs: how many (token, expert) pairs there are, where known (a step has no more tiles than pairs). Per place: out[place] = w[expert] a[row]; gated: act(gate a) * (up a), w [experts, 2 N, K] holding gate and up rows in
     alternating groups of `group`. row = pair // gather_div, or the place itself where gather_div is 0."""
     from .recurrent import GATE_ACTIVATIONS
     require(w, "w", _FLOATS, (None, None, None))
@@ -341,8 +345,15 @@ def moe_gemm(a: torch.Tensor, w: torch.Tensor, gated: bool, group: int, out: tor
                                                                                   and out.dtype == torch.bfloat16))):
         check(entry("llme_gemm_bf16_grouped")(ptr(a), ptr(w), ptr(out), code(out.dtype), 1 if gated else 0, rows_w, K, tile,
                                               cap // tile, ptr(tile_expert), ptr(n_tiles), ptr(place_pair) if gather_div else None,
-                                              max(gather_div, 1), a.shape[0], E, 0, stream()), "moe_gemm")
+                                              max(gather_div, 1), a.shape[0], E, 0, 0, stream()), "moe_gemm")
         return
+    if moe_few_rows(tile, a, w, out, gated, group, activation, choices):
+        check(entry("llme_gemm_few_grouped")(ptr(a), ptr(w), ptr(out), 1 if gated else 0, N, K, GATE_ACTIVATIONS[activation],
+                                             min(cap // tile, pairs or cap), ptr(tile_expert), ptr(n_tiles), ptr(place_pair), int(gather_div),
+                                             ptr(pair_scale), stream()), "moe_gemm")
+        return
+    if pair_scale is not None:
+        raise KernelError("moe_gemm: weights on the experts' input need the kernels for few rows or the gated epilogue")
     check(entry("llme_moe_gemm")(ptr(a), code(a.dtype), ptr(w), 1 if gated else 0, code(w.dtype), ptr(out), code(out.dtype),
                                  ptr(place_pair), ptr(tile_expert), ptr(n_tiles), tile, cap // tile, int(gather_div), N, K,
                                  int(group), GATE_ACTIVATIONS[activation], stream()), "moe_gemm")
@@ -399,3 +410,64 @@ def moe_combine(y: torch.Tensor, pair_place: torch.Tensor, wts: torch.Tensor | N
     check(entry("llme_moe_combine")(ptr(y), ptr(pair_place), ptr(wts), ptr(out), T, top, H, 1 if accumulate else 0, ptr(shared),
                                     ptr(shared_gate), ld_gate, stream()),
           "moe_combine")
+
+
+# --- the router of few tokens, the sum with the norm behind ------------------------------------
+declare("llme_moe_decide", [_vp, _vp, _i, _i, _i, _i, _i, _f, _i, _i, _vp, _i, _vp, _i, _i, _vp, _vp, _vp, _vp, _vp])
+declare("llme_moe_combine_norm", [_vp, _vp, _vp, _i, _vp, _vp, _i, _i, _vp, _i, _vp, _vp, _i, _i, _i, _f, _f, _vp])
+MOE_DECIDE_TOKENS, MOE_DECIDE_ROWS, MOE_DECIDE_TOP = 16, 128, 32     # what the one workgroup holds
+
+
+def moe_decide_fits(x: torch.Tensor, w: torch.Tensor, top: int, choices=None) -> bool:
+    from .choices import DEFAULT
+    return ((choices or DEFAULT).fast_gemm and x.shape[0] <= MOE_DECIDE_TOKENS and w.dim() == 2 and w.shape[0] <= MOE_DECIDE_ROWS
+            and top <= MOE_DECIDE_TOP and x.dtype == torch.bfloat16 and w.dtype == torch.bfloat16 and x.shape[1] % 8 == 0
+            and x.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0)
+
+
+def moe_decide(x: torch.Tensor, w: torch.Tensor, experts: int, top: int, scale: float, renormalize: bool, logits: torch.Tensor,
+               wts: torch.Tensor, tile: int, place_pair: torch.Tensor, pair_place: torch.Tensor, tile_expert: torch.Tensor,
+               n_tiles: torch.Tensor, scoring: str = "softmax") -> None:
+    """logits[t, :rows] = x w^T (32-bit sums) for w [rows, K], rows = experts or one more (a gate's row, which takes no part in the
+    choice), then moe_route on the first `experts` and moe_plan, in one launch; bfloat16, few tokens."""
+    if scoring not in ("softmax", "sigmoid"):
+        raise KernelError(f"moe_decide: scoring {scoring!r} is neither 'softmax' nor 'sigmoid'")
+    require(x, "x", torch.bfloat16, (None, None))
+    T, K = x.shape
+    require(w, "w", torch.bfloat16, (None, K))
+    require(logits, "logits", torch.float32, (T, None))
+    require(wts, "wts", torch.float32, (T, top))
+    cap = moe_capacity(T * top, experts, tile)
+    require(place_pair, "place_pair", torch.int32, (cap,))
+    require(pair_place, "pair_place", torch.int32, (T * top,))
+    require(tile_expert, "tile_expert", torch.int32, (cap // tile,))
+    require(n_tiles, "n_tiles", torch.int32, (1,))
+    check(entry("llme_moe_decide")(ptr(x), ptr(w), T, K, w.shape[0], experts, top, float(scale), 1 if renormalize else 0,
+                                   1 if scoring == "sigmoid" else 0, ptr(logits), logits.shape[1], ptr(wts), tile, cap, ptr(place_pair),
+                                   ptr(pair_place), ptr(tile_expert), ptr(n_tiles), stream()), "moe_decide")
+
+
+def moe_combine_norm(y: torch.Tensor, pair_place: torch.Tensor, wts: torch.Tensor | None, top: int, shared: torch.Tensor | None,
+                     shared_gate: torch.Tensor | None, weight: torch.Tensor, h: torch.Tensor, eps: float, x_out: torch.Tensor | None,
+                     scale: float = 1.0, clear_shared: bool = False) -> None:
+    """h += scale * (weight * c / rms(c)), c[t] = sum_k wts[t, k] y[place of (t, k)] + sigmoid(shared_gate[t]) shared[t] (shared None:
+    nothing; shared_gate None: shared as it is); x_out (or None): the updated rows in its type. clear_shared: shared is zeros after."""
+    require(h, "h", torch.float32, (None, None))
+    T, H = h.shape
+    require(y, "y", torch.float32, (None, H))
+    require(pair_place, "pair_place", torch.int32, (T * top,))
+    if wts is not None:
+        require(wts, "wts", torch.float32, (T, top))
+    ld_gate = 0
+    if shared is not None:
+        require(shared, "shared", torch.float32, (T, H))
+        if shared_gate is not None:
+            from .recurrent import _cols
+            ld_gate = _cols(shared_gate, "shared_gate", torch.float32, T, 1)
+    require(weight, "weight", _FLOATS, (H,))
+    if x_out is not None:
+        require(x_out, "x_out", _FLOATS, (T, H))
+    check(entry("llme_moe_combine_norm")(ptr(y), ptr(pair_place), ptr(wts), top, ptr(shared), ptr(shared_gate) if ld_gate else None, ld_gate,
+                                         1 if clear_shared else 0, ptr(weight), code(weight.dtype), ptr(h), ptr(x_out),
+                                         code(x_out.dtype) if x_out is not None else 0, T, H, float(eps), float(scale), stream()),
+          "moe_combine_norm")

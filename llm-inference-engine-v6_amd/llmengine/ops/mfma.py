@@ -53,6 +53,9 @@ def gemm_bf16(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, accumulate: b
           "gemm_bf16")
 
 
+FEW_ROWS = 16                       # rows up to which gated products stream their weights (csrc/gemm_few_rows.hip)
+
+
 def gemm_gated(x: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tensor, group: int, scratch,
                choices: KernelChoices | None = None, activation: str = "silu") -> None:
     """out [T, FF] = act(x Wg^T) * (x Wu^T) (act SiLU unless named otherwise), the gate and up rows interleaved in groups of `group`
@@ -63,6 +66,16 @@ def gemm_gated(x: torch.Tensor, w_gate_up: torch.Tensor, out: torch.Tensor, grou
     if ((choices or DEFAULT).fast_gemm and group == 16 and out.dtype == torch.bfloat16 and (2 * FF) % 32 == 0
             and activation in ("silu", "relu", "gelu_tanh")
             and x.dtype == torch.bfloat16 and gemm_bf16_supported(x, w_gate_up, out, False)):
+        if T <= FEW_ROWS and w_gate_up.shape[-1] % 8 == 0:
+            # (few rows: the weights streamed once, no tile of rows)
+            from .recurrent import GATE_ACTIVATIONS
+            require(x, "x", torch.bfloat16, (T, None))
+            n_rows, _ = kernels._require_weight(w_gate_up, "w_gate_up", torch.bfloat16, x.shape[1])
+            if n_rows != 2 * FF:
+                raise kernels.KernelError(f"gemm_gated: {n_rows} weight rows for {FF} units")
+            check(entry("llme_gemm_few_gated")(ptr(x), ptr(w_gate_up), ptr(out), T, FF, x.shape[1], 1 if kernels.is_blocked(w_gate_up) else 0,
+                                               GATE_ACTIVATIONS[activation], stream()), "gemm_gated")
+            return
         r = tail_rows(T, choices)
         mode = activation if activation in ("relu", "gelu_tanh") else True
         if r:

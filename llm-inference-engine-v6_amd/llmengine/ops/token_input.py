@@ -42,3 +42,25 @@ def token_gate(z: torch.Tensor, table: torch.Tensor, col: int, tokens: torch.Ten
         raise KernelError(f"token_gate: columns {col} .. {col + n} of a table of {table.shape[1]}")
     check(entry("llme_token_gate")(ptr(z), ld, ptr(table), code(table.dtype), table.shape[1], int(col), ptr(tokens), ptr(out),
                                    code(out.dtype), T, n, stream()), "token_gate")
+
+
+def gemm_token_gate(x: torch.Tensor, w: torch.Tensor, table: torch.Tensor, col: int, tokens: torch.Tensor, out: torch.Tensor,
+                    choices=None) -> bool:
+    """token_gate of z = x w^T in one launch, for few rows of a bfloat16 model (returns False, with nothing done, for any other
+    step): x [T, K], w [n, K] (row-major or blocked), out [T, n]."""
+    from .choices import DEFAULT
+    from .mfma import FEW_ROWS, gemm_bf16_supported
+    T, n = out.shape
+    if not ((choices or DEFAULT).fast_gemm and T <= FEW_ROWS and out.dtype == torch.bfloat16 and table.dtype == torch.bfloat16
+            and x.dtype == torch.bfloat16 and gemm_bf16_supported(x, w, out, False)):
+        return False
+    require(x, "x", torch.bfloat16, (T, None))
+    K = x.shape[1]
+    n_rows, _ = _require_weight(w, "w", torch.bfloat16, K)
+    require(table, "table", torch.bfloat16, (None, None))
+    require(tokens, "tokens", torch.int32, (T,))
+    if n_rows != n or not 0 <= col <= table.shape[1] - n:
+        raise KernelError(f"gemm_token_gate: {n_rows} rows, columns {col} .. {col + n} of a table of {table.shape[1]}")
+    check(entry("llme_gemm_few_token_gate")(ptr(x), ptr(w), ptr(out), T, n, K, 1 if is_blocked(w) else 0, ptr(table), table.shape[1], int(col),
+                                            ptr(tokens), stream()), "gemm_token_gate")
+    return True

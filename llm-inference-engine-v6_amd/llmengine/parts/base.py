@@ -278,6 +278,12 @@ class FeedForward(Part):
     def fuses_norm(self, h: torch.Tensor, norm: "Norm", step) -> bool:
         return False
 
+    def fuses_output_norm(self, h: torch.Tensor, step) -> bool:
+        """True if, for this step, the part wants to do itself what a block does with its result where the norm stands behind
+        the sublayer: `forward_normed(x, step, h, weight, eps, scale, x_out)` adds scale * (weight * y / rms(y)) of its result
+        y into the stream h and leaves the updated rows in x_out (or nothing where x_out is None)."""
+        return False
+
     def forward(self, x: torch.Tensor, step, out: torch.Tensor, accumulate: bool) -> None:
         raise NotImplementedError
 

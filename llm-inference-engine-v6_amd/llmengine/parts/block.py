@@ -224,8 +224,14 @@ class OutputNormBlock(Block):
         last = 2 if self.token_input is not None else 1 if self.feed_forward is not None else 0
         self._join(y, self.mixer_norm, h, x if hand_on or last > 0 else h, add, c, scales[0])
         if self.feed_forward is not None:
-            self.feed_forward.forward(x, step, y, add)
-            self._join(y, self.ffn_norm, h, x if hand_on or last > 1 else h, add, c, scales[1])
+            copy = x if hand_on or last > 1 else h
+            rms = self.ffn_norm.fused_rms()
+            if rms is not None and self.feed_forward.fuses_output_norm(h, step):
+                self.feed_forward.forward_normed(x, step, h, scales[1] if scales[1] is not None else rms[0], rms[1], c,
+                                                 copy if copy is not h else None)
+            else:
+                self.feed_forward.forward(x, step, y, add)
+                self._join(y, self.ffn_norm, h, copy, add, c, scales[1])
         if self.token_input is not None:
             self.token_input.forward(x, step, y, add)
             self._join(y, self.token_input.norm, h, x if hand_on else h, add)

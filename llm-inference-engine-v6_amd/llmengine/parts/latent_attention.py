@@ -149,10 +149,8 @@ class LatentAttention(Mixer):
             ol = ol.view(n, T, R)
             ops.latent.latent_attention_mfma(qa, qr, rows, ol, step, table, n, R, self.scale, self.window, head_major=True,
                                             **extras)
-            oh = step.buffer("latent.oh", (n, T, dv), act)
-            ops.latent.heads_gemm(ol, self.w_uv, oh)
             o = step.buffer("latent.o", (T, n * dv), act)
-            ops.latent.heads_to_rows(oh, o)
+            ops.latent.heads_gemm(ol, self.w_uv, o)
             ops.gemm(o, self.w_o, out, accumulate, fixed_order=step.fixed_order, choices=step.choices)
             return
         if fast:

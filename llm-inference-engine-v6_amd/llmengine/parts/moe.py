@@ -33,6 +33,7 @@ from .registry import register_part
 
 class MixtureOfExperts(FeedForward):
     graph_safe = True
+    ADDED_ROWS = 64             # steps of up to this many rows add the parts of the shared expert's last product
 
     def __init__(self, hidden_size: int, intermediate_size: int, experts: int, top: int, scale: float = 1.0,
                  renormalize: bool = False, activation: str = "silu", shared: FeedForward | None = None,
@@ -86,10 +87,13 @@ class MixtureOfExperts(FeedForward):
         # The router's matrix as the file has it: bfloat16 entries times the bfloat16 input are exact in 32-bit, so the
         # matrix-core product with its 32-bit sums is the 32-bit product; the 32-bit model widens it like everything else.
         if self.router != "table":
+            # (twice where the product's kernels want another layout: steps of few tokens read it row by row)
+            parts = [get("router")] + ([get("shared.sg")] if self.shared_gate else [])
+            self.w_router_rows = placement.place(torch.cat(parts) if self.shared_gate else parts[0])
             if self.shared_gate:
-                self.w_router, self.route_columns = stack_rows([get("router"), get("shared.sg")], placement)
+                self.w_router, self.route_columns = stack_rows(parts, placement)
             else:
-                self.w_router, self.route_columns = placement.place(get("router")), self.experts
+                self.w_router, self.route_columns = self.w_router_rows, self.experts
         else:
             self.table = placement.place(get("table"))
             if int(self.table.min()) < 0 or int(self.table.max()) >= self.experts:
@@ -107,21 +111,61 @@ class MixtureOfExperts(FeedForward):
         self.w_down = torch.stack([placement.place(get(f"{n}.down"), dtype) for n in names]).contiguous()
 
     def forward(self, x, step, out, accumulate):
+        y, pair_place, wts, logits = self._experts(x, step)
+        T, H = x.shape
+        f32 = torch.float32
+        shared = dict()
+        if self.shared_gate:
+            rows = step.buffer("moe.shared", (T, H), f32)
+            self.shared.forward(x, step, rows, False)
+            shared = dict(shared=rows, shared_gate=logits[:, self.experts:self.experts + 1])
+        elif self.shared is not None:
+            self.shared.forward(x, step, out, accumulate)
+            accumulate = True
+        ops.moe_combine(y, pair_place, wts, out, accumulate, top=self.top, **shared)
+
+    def fuses_output_norm(self, h, step):
+        return self.hidden_size % 4 == 0 and self.hidden_size <= ops.latent.MOE_COMBINE_NORM_MAX
+
+    def forward_normed(self, x, step, h, weight, eps, scale, x_out):
+        y, pair_place, wts, logits = self._experts(x, step)
+        rows = gate = None
+        add = False
+        if self.shared is not None:
+            T, H = x.shape
+            # few rows: the shared expert's last product is cut over k, its parts added into zeros that the sum leaves as zeros
+            add = T <= self.ADDED_ROWS and not step.fixed_order and step.act_dtype == torch.bfloat16
+            rows = step.buffer("moe.shared_sum" if add else "moe.shared", (T, H), torch.float32)
+            if add and not step.extra.get("moe.shared_sum is clear"):
+                ops.clear(rows)
+                step.extra["moe.shared_sum is clear"] = True
+            self.shared.forward(x, step, rows, add)
+            gate = logits[:, self.experts:self.experts + 1] if self.shared_gate else None
+        ops.latent.moe_combine_norm(y, pair_place, wts, self.top, rows, gate, weight, h, eps, x_out, scale, clear_shared=add)
+
+    def _experts(self, x, step):
+        """The experts' results by place: (y [places, H], pair -> place, the pairs' weights or None, the router's logits)."""
         T, H = x.shape
         E, top, FF = self.experts, self.top, self.intermediate_size
         i32, f32 = torch.int32, torch.float32
         ids, wts = step.buffer("moe.ids", (T, top), i32), step.buffer("moe.weights", (T, top), f32)
-        if self.router == "table":
-            ops.window.table_route(self.table, step.tokens, ids, wts)
-        else:
-            logits = step.buffer("moe.logits", (T, self.route_columns), f32)
-            ops.gemm(x, self.w_router, logits, choices=step.choices)
-            ops.moe_route(logits[:, :E], top, self.scale, self.renormalize, ids, wts, scoring=self.router)
+        logits = None
         tile = ops.latent.moe_tile(x, self.w_gate_up, T * top, E, self.group, step.choices)
         cap = ops.moe_capacity(T * top, E, tile)
         place_pair, pair_place = step.buffer("moe.place_pair", (cap,), i32), step.buffer("moe.pair_place", (T * top,), i32)
         tile_expert, n_tiles = step.buffer("moe.tile_expert", (cap // tile,), i32), step.buffer("moe.tiles", (1,), i32)
-        ops.moe_plan(ids, E, tile, place_pair, pair_place, tile_expert, n_tiles)
+        if self.router == "table":
+            ops.window.table_route(self.table, step.tokens, ids, wts)
+            ops.moe_plan(ids, E, tile, place_pair, pair_place, tile_expert, n_tiles)
+        else:
+            logits = step.buffer("moe.logits", (T, self.route_columns), f32)
+            if ops.latent.moe_decide_fits(x, self.w_router_rows, top, step.choices):
+                ops.latent.moe_decide(x, self.w_router_rows, E, top, self.scale, self.renormalize, logits, wts, tile, place_pair,
+                                      pair_place, tile_expert, n_tiles, scoring=self.router)
+            else:
+                ops.gemm(x, self.w_router, logits, choices=step.choices)
+                ops.moe_route(logits[:, :E], top, self.scale, self.renormalize, ids, wts, scoring=self.router)
+                ops.moe_plan(ids, E, tile, place_pair, pair_place, tile_expert, n_tiles)
         act = step.buffer("moe.act", (cap, FF), step.act_dtype)
         if self.activation == "swish_clamped" and ops.latent.moe_gemm_clamped(x, self.w_gate_up, self.group, act, place_pair,
                                                                              tile_expert, n_tiles, tile, top, self.limit, 1.702,
@@ -131,6 +175,9 @@ class MixtureOfExperts(FeedForward):
                 x, self.w_gate_up, self.group, act, place_pair, tile_expert, n_tiles, tile, top, 0.0, 1.0, step.choices,
                 pair_scale=wts.view(-1)):
             pass                            # (a place's sums times its pair's weight, then the activation, in the product's epilogue)
+        elif self.weight_on == "input" and ops.latent.moe_few_rows(tile, x, self.w_gate_up, act, True, self.group, self.activation, step.choices):
+            ops.moe_gemm(x, self.w_gate_up, True, self.group, act, place_pair, tile_expert, n_tiles, tile, top, self.activation,
+                         step.choices, pairs=T * top, pair_scale=wts.view(-1))
         elif self.weight_on == "input":
             # the gate and up sums as 32-bit rows, each row times its pair's weight, then the activation, in one pass
             gu = step.buffer("moe.gate_up", (cap, 2 * FF), f32)
@@ -143,18 +190,10 @@ class MixtureOfExperts(FeedForward):
             ops.window.gated_bias_act(gu, act, self.group, "swish_clamped", None, self.limit, 1.702)
         else:
             ops.moe_gemm(x, self.w_gate_up, True, self.group, act, place_pair, tile_expert, n_tiles, tile, top, self.activation,
-                         step.choices)
+                         step.choices, pairs=T * top)
         y = step.buffer("moe.y", (cap, H), f32)
-        ops.moe_gemm(act, self.w_down, False, 0, y, place_pair, tile_expert, n_tiles, tile, 0, "silu", step.choices)
-        shared = dict()
-        if self.shared_gate:
-            rows = step.buffer("moe.shared", (T, H), f32)
-            self.shared.forward(x, step, rows, False)
-            shared = dict(shared=rows, shared_gate=logits[:, E:E + 1])
-        elif self.shared is not None:
-            self.shared.forward(x, step, out, accumulate)
-            accumulate = True
-        ops.moe_combine(y, pair_place, wts if self.weight_on == "output" else None, out, accumulate, top=top, **shared)
+        ops.moe_gemm(act, self.w_down, False, 0, y, place_pair, tile_expert, n_tiles, tile, 0, "silu", step.choices, pairs=T * top)
+        return y, pair_place, wts if self.weight_on == "output" else None, logits
 
 
 register_part("feed_forward", "mixture_of_experts", MixtureOfExperts)

@@ -51,8 +51,9 @@ class TokenInput(Part):
     def forward(self, x: torch.Tensor, step, out: torch.Tensor, accumulate: bool) -> None:
         """out [T, H] (32-bit) (+)= P (gelu(G x) * e), in front of the norm."""
         T, d = x.shape[0], self.table.dim
-        z = step.buffer("token_input.gate", (T, d), torch.float32)
-        ops.gemm(x, self.w_gate, z, choices=step.choices)
         g = step.buffer("token_input.gated", (T, d), step.act_dtype)
-        ops.token_input.token_gate(z, self.table.weight, self.index * d, step.tokens, g)
+        if not ops.token_input.gemm_token_gate(x, self.w_gate, self.table.weight, self.index * d, step.tokens, g, choices=step.choices):
+            z = step.buffer("token_input.gate", (T, d), torch.float32)
+            ops.gemm(x, self.w_gate, z, choices=step.choices)
+            ops.token_input.token_gate(z, self.table.weight, self.index * d, step.tokens, g)
         ops.gemm(g, self.w_proj, out, accumulate, fixed_order=step.fixed_order, choices=step.choices)

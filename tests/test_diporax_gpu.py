@@ -318,7 +318,7 @@ def test_the_joined_norm_and_its_gate(T, width):
         assert bool((wide[:, :8] == 7).all()) and bool((wide[:, 8 + width:] == 7).all())
 
 
-@pytest.mark.parametrize("H", [28, 64, 2048, 3000])
+@pytest.mark.parametrize("H", [28, 64, 2048, 3000, 4096, 8192, 8200])
 def test_a_normed_embedding_and_the_tokens_gate(H):
     from llmengine import ops
     g = torch.Generator().manual_seed(H)
