@@ -17,6 +17,10 @@ the expert's two input products: their 32-bit sums are multiplied by it in front
 names the experts of every token id, each weighing 1 / top. `activation="swish_clamped"` with `limit`:
 g = min(gate, limit), u = clamp(up, -limit, limit), the expert's inner value is g sigmoid(1.702 g) (u + 1).
 
+A step of few tokens makes its router's product, the choice and the plan in one launch and streams the experts' weights in
+tiles of 16 rows; where the norm stands behind the layer, the sum of the experts' results, the norm and the sum into the
+stream are one kernel (`forward_normed`).
+
 On the device the (token, expert) pairs are grouped by expert into tiles of rows, and two grouped products
 (gate/up with the activation, then down) run over the tiles; nothing of the routing comes to the host, so
 a step's launches do not depend on what the tokens choose.
